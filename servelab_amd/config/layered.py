@@ -28,6 +28,25 @@ def _section(cfg: Dict[str, Any], key: str, where: str, required=True) -> Option
     return value
 
 
+def weights_owner(entries: List[Any], i: int):
+    """(the layer whose tensors layer i runs, or None for its own; layer i's entry, with what it leaves
+    out taken from the owner's).  ``weights_of`` is followed through layers that borrow in turn."""
+    where, entry = f"layers[{i}]", entries[i]
+    if not isinstance(entry, dict):
+        raise ConfigError(f"config.json: {where} must be an object")
+    if entry.get("weights_of") is None:
+        return None, entry
+    owner, seen = read_key(entry, "weights_of", kind=int), {i}
+    while True:
+        if not 0 <= owner < len(entries) or owner in seen or not isinstance(entries[owner], dict):
+            raise ConfigError(f"config.json: {where}: weights_of must lead to another layer that has tensors of its own")
+        if entries[owner].get("weights_of") is None:
+            break
+        seen.add(owner)
+        owner = read_key(entries[owner], "weights_of", kind=int)
+    return owner, dict(entries[owner], **{k: v for k, v in entry.items() if k != "weights_of"})
+
+
 @dataclass(frozen=True)
 class WindowConfig:
     """Query i sees key j <= i when i - j < size or j < keep_first; size 0: every j <= i."""

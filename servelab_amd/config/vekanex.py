@@ -19,7 +19,7 @@ Nothing here is a default for a size or a constant of the model.
 from dataclasses import dataclass, field
 from typing import Any, Dict, List, Optional
 
-from .layered import _section
+from .layered import _section, weights_owner
 from .model import ConfigError, read_key
 
 
@@ -207,24 +207,9 @@ class VekanexConfig:
             except Exception:
                 shapes = None                     # a folder without weights: the ranks must be keys
         layers = []
-        for i, entry in enumerate(entries):
+        for i in range(len(entries)):
             where = f"layers[{i}]"
-            if not isinstance(entry, dict):
-                raise ConfigError(f"config.json: {where} must be an object")
-            owner = entry.get("weights_of")
-            if owner is not None:
-                # the layer whose tensors these are, through any layers that borrow them in turn
-                owner, seen = read_key(entry, "weights_of", kind=int), {i}
-                while True:
-                    if not 0 <= owner < len(entries) or owner in seen or not isinstance(entries[owner], dict):
-                        raise ConfigError(f"config.json: {where}: weights_of must lead to another layer "
-                                          "that has tensors of its own")
-                    if entries[owner].get("weights_of") is None:
-                        break
-                    seen.add(owner)
-                    owner = read_key(entries[owner], "weights_of", kind=int)
-                # what the entry leaves out it takes from the owner's
-                entry = dict(entries[owner], **{k: v for k, v in entry.items() if k != "weights_of"})
+            owner, entry = weights_owner(entries, i)
             kind = read_key(entry, "type", kind=str)
             prefix = f"l{i if owner is None else owner}.mix."
             mixer = _read_mixer(kind, _section(entry, "mixer", where), prefix, shapes, where)

@@ -476,7 +476,8 @@ struct NormFusion {
   // that do (N = 5120 on 256 CUs: 512 tiles of 10 rows instead of 320 of 16).  Other forms: 16.
   int th;
   int pair_x;                // at most 8 rows and one tile a workgroup: a load of x takes two k-steps (see stream_k2)
-  int gate_act;              // gated forms: the activation of the gate (common.h: 1 silu, 2 relu)
+  int gate_act;              // gated forms: the activation of the gate (common.h: 1 silu, 2 relu); plain form: the
+                             // activation of the result (0: none)
 };
 
 // Rotary embedding and the write to the cache pages fused into the q/k/v
@@ -794,8 +795,10 @@ __global__ __launch_bounds__(64 * WAVES) void gemm_skinny_kernel(
         for (int o = 8; o > 0; o >>= 1) sq += __shfl_xor(sq, o, 64);     // over the 16 columns of row m
         if (n_local == 0) F.out_parts[(size_t)tile * 16 + m] = sq;
       } else if (live) {
-        if (out_f32) ((float*)y)[(size_t)m * N + n] = s;
-        else ((__bf16*)y)[(size_t)m * N + n] = (__bf16)s;
+        if (!CONSUMER && F.gate_act) s = sl_act(s, F.gate_act);
+        const size_t at = !CONSUMER && F.y_tiled ? (size_t)(n / 32) * (M * 32) + m * 32 + n % 32 : (size_t)m * N + n;
+        if (out_f32) ((float*)y)[at] = s;
+        else ((__bf16*)y)[at] = (__bf16)s;
       }
     }
   }
@@ -821,7 +824,7 @@ extern "C" const char* sl_gemm_skinny(const void* x, const void* wt, const float
                                       const float* in_parts, int in_nparts, float eps,
                                       const int* rows, float* resid, const float* next_w,
                                       float* out_parts, const RopeStore* rope, int pair_tiles,
-                                      int x_tiled, int y_tiled, int th, int pair_x, hipStream_t stream) {
+                                      int x_tiled, int y_tiled, int th, int pair_x, int act, hipStream_t stream) {
   SL_CHECK(M >= 0 && N > 0 && K > 0, "gemm_skinny: sizes must be positive");
   SL_CHECK(M <= 16, "gemm_skinny: at most 16 rows");
   SL_CHECK(K % 32 == 0, "gemm_skinny: K must be a multiple of 32");
@@ -835,6 +838,8 @@ extern "C" const char* sl_gemm_skinny(const void* x, const void* wt, const float
   SL_CHECK(!consumer || in_nparts <= 32 * SL_MAX_PARTS_PER_THREAD,
            "gemm_skinny: un-normalised rows of more than 8192 values");
   SL_CHECK(rows == nullptr || consumer, "gemm_skinny: a row gather belongs to a consumer");
+  SL_CHECK(!act || (!gated && !consumer && !producer && !out_f32 && rope == nullptr && act >= SL_ACT_SILU && act <= SL_ACT_GELU_TANH),
+           "gemm_skinny: an activation goes with a plain product in the activation dtype");
   SL_CHECK(!producer || (next_w != nullptr && out_parts != nullptr && !gated && !out_f32),
            "gemm_skinny: a producer needs the next gain and a parts buffer, and is neither gated nor float");
   SL_CHECK(th == 16 || (producer && th >= 8 && th < 16 && th % 2 == 0),
@@ -845,9 +850,9 @@ extern "C" const char* sl_gemm_skinny(const void* x, const void* wt, const float
   const __bf16* ww = (const __bf16*)wt;
   SL_CHECK(x_tiled >= 0 && (x_tiled == 0 || rows != nullptr || x_tiled == M),
            "gemm_skinny: x tiled by k-step has as many rows as the product, or rows are picked from it");
-  SL_CHECK(!y_tiled || (gated && (N / 2) % 32 == 0) || (resid != nullptr && N % 32 == 0),
-           "gemm_skinny: a tiled result is a gated one or a producer's, of a multiple of 32 columns");
-  const NormFusion F{in_parts, in_nparts, eps, rows, resid, next_w, out_parts, x_tiled, y_tiled, th, pair_x, gated};
+  SL_CHECK(!y_tiled || (gated && (N / 2) % 32 == 0) || ((resid != nullptr || act) && N % 32 == 0),
+           "gemm_skinny: a tiled result is a gated, an activated or a producer's, of a multiple of 32 columns");
+  const NormFusion F{in_parts, in_nparts, eps, rows, resid, next_w, out_parts, x_tiled, y_tiled, th, pair_x, gated ? gated : act};
   const bool few = in_nparts <= 32 * 8;
   if (rope != nullptr) {
     const RopeStore R = *rope;
@@ -1234,6 +1239,7 @@ __global__ __launch_bounds__(512) void gemm_wide_kernel(
 #pragma unroll
         for (int wv = 0; wv < WAVES; ++wv) sum += red[wv][b][m_local + 16 * (n_local / 4)][n_local % 4];
         if (bias != nullptr) sum += bias[n];
+        if (gate_act) sum = sl_act(sum, gate_act);
         if (out_f32) ((float*)y)[(size_t)m * N + n] = sum;
         else ((__bf16*)y)[(size_t)m * N + n] = (__bf16)sum;
       }
@@ -1242,13 +1248,15 @@ __global__ __launch_bounds__(512) void gemm_wide_kernel(
 }
 
 extern "C" const char* sl_gemm_wide(const void* x, const void* wt, const float* bias, void* y,
-                                    int M, int N, int K, int out_f32, int gated,
+                                    int M, int N, int K, int out_f32, int gated, int act,
                                     hipStream_t stream) {
   SL_CHECK(M > 0 && N > 0 && K > 0, "gemm_wide: sizes must be positive");
   SL_CHECK(M <= 64, "gemm_wide: at most 64 rows");
   SL_CHECK(K % 32 == 0, "gemm_wide: K must be a multiple of 32");
   SL_CHECK(!gated || (N % 16 == 0 && !out_f32),
            "gemm_wide: the gated form needs N % 16 == 0, activation output");
+  SL_CHECK(!act || (!gated && !out_f32 && act >= SL_ACT_SILU && act <= SL_ACT_GELU_TANH),
+           "gemm_wide: an activation goes with a plain product in the activation dtype");
   SL_CHECK(((uintptr_t)x % 16) == 0 && ((uintptr_t)wt % 16) == 0,
            "gemm_wide: x and W must be 16-byte aligned");
   const dim3 grid(((N + 15) / 16 + 1) / 2);
@@ -1258,8 +1266,8 @@ extern "C" const char* sl_gemm_wide(const void* x, const void* wt, const float* 
     if (M <= 32) gemm_wide_kernel<2, true><<<grid, 512, 0, stream>>>(xx, ww, bias, y, M, N, K, 0, gated);
     else gemm_wide_kernel<4, true><<<grid, 512, 0, stream>>>(xx, ww, bias, y, M, N, K, 0, gated);
   } else {
-    if (M <= 32) gemm_wide_kernel<2, false><<<grid, 512, 0, stream>>>(xx, ww, bias, y, M, N, K, out_f32, 0);
-    else gemm_wide_kernel<4, false><<<grid, 512, 0, stream>>>(xx, ww, bias, y, M, N, K, out_f32, 0);
+    if (M <= 32) gemm_wide_kernel<2, false><<<grid, 512, 0, stream>>>(xx, ww, bias, y, M, N, K, out_f32, act);
+    else gemm_wide_kernel<4, false><<<grid, 512, 0, stream>>>(xx, ww, bias, y, M, N, K, out_f32, act);
   }
   return sl_launch_status();
 }
@@ -1276,7 +1284,7 @@ extern "C" const char* sl_gemm_wide(const void* x, const void* wt, const float* 
 template <int MB, int NT, int KC, int WAVES>
 __global__ __launch_bounds__(64 * WAVES) void gemm_mid_kernel(
     const __bf16* __restrict__ x, const __bf16* __restrict__ wt, const float* __restrict__ bias,
-    void* __restrict__ y, int M, int N, int K, int out_f32, int gated, int KS) {
+    void* __restrict__ y, int M, int N, int K, int out_f32, int gated, int KS, int act) {
   constexpr int THREADS = 64 * WAVES;
   // chunks of W in flight or in use (LDS holds as many of x): three for the workgroups of eight
   // wavefronts where the registers and LDS allow it (gate/up of the 7B shape at 64 rows: 52 -> 49 us);
@@ -1519,6 +1527,10 @@ __global__ __launch_bounds__(64 * WAVES) void gemm_mid_kernel(
 #pragma unroll
       for (int r = 0; r < 4; ++r)
         if (bias != nullptr && n + r < N) v[r] += bias[n + r];
+      if (act) {
+#pragma unroll
+        for (int r = 0; r < 4; ++r) v[r] = sl_act(v[r], act);
+      }
       if (whole && out_f32) {
         *(f32x4*)((float*)y + (size_t)m * N + n) = v;
       } else if (whole) {
@@ -1554,7 +1566,7 @@ __global__ void splitk_reduce_kernel(const float* __restrict__ part, const float
 // for the reader to add (and the bias with them).
 extern "C" const char* sl_gemm_mid(const void* x, const void* wt, const float* bias, void* y,
                                    int M, int N, int K, int out_f32, int gated, int ks,
-                                   int wide_min_wgs, int num_cus, float* part, hipStream_t stream) {
+                                   int wide_min_wgs, int num_cus, float* part, int act, hipStream_t stream) {
   SL_CHECK(M > 0 && N > 0 && K > 0, "gemm_mid: sizes must be positive");
   SL_CHECK(M <= 128, "gemm_mid: at most 128 rows");
   SL_CHECK(K % 32 == 0, "gemm_mid: K must be a multiple of 32");
@@ -1563,6 +1575,8 @@ extern "C" const char* sl_gemm_mid(const void* x, const void* wt, const float* b
   SL_CHECK(y != nullptr || ks > 1, "gemm_mid: no output");
   SL_CHECK(!gated || (ks == 1 && N % 16 == 0 && !out_f32),
            "gemm_mid: the gated form needs ks == 1, N % 16 == 0, activation output");
+  SL_CHECK(!act || (!gated && ks == 1 && !out_f32 && act >= SL_ACT_SILU && act <= SL_ACT_GELU_TANH),
+           "gemm_mid: an activation goes with an unsplit plain product in the activation dtype");
   SL_CHECK(((uintptr_t)x % 16) == 0 && ((uintptr_t)wt % 16) == 0,
            "gemm_mid: x and W must be 16-byte aligned");
   const int ntiles = (N + 15) / 16;
@@ -1589,7 +1603,7 @@ extern "C" const char* sl_gemm_mid(const void* x, const void* wt, const float* b
   // alone); the workgroups of eight wavefronts share out a chunk of x evenly for even counts only
   const int mb = (M + 15) / 16;
 #define SL_MID(MB_, WAVES_) gemm_mid_kernel<MB_, 2, 4, WAVES_><<<grid, 64 * WAVES_, 0, stream>>>( \
-    xx, ww, bias, dst, M, N, K, out_f32, gated, ks)
+    xx, ww, bias, dst, M, N, K, out_f32, gated, ks, act)
   if (wide) {
     if (mb <= 2) SL_MID(2, 8);
     else if (mb <= 4) SL_MID(4, 8);

@@ -313,15 +313,15 @@ extern "C" const char* sl_add_into(float* resid, const void* delta, long long n,
 }
 
 // RMS norm on a sublayer's output: resid (float, in place) += mult * y * rsqrt(mean(y^2) + eps) * w,
-// and the stream's new rows in the activation type for the sublayer that reads them next.  y == nullptr:
-// only those rows.  One block per row; sums and the stream in float.
+// and the stream's new rows in the activation type for the sublayer that reads them next (out == nullptr:
+// they are not wanted).  y == nullptr: only those rows.  One block per row; sums and the stream in float.
 __global__ void add_postnorm_kernel(float* __restrict__ resid, const act_t* __restrict__ y,
                                     const float* __restrict__ w, act_t* __restrict__ out, int H, float eps,
                                     float mult) {
   __shared__ float scratch[16];
   const size_t r = blockIdx.x;
   float* x = resid + r * H;
-  act_t* o = out + r * H;
+  act_t* o = out != nullptr ? out + r * H : nullptr;
   if (y == nullptr) {
     for (int i = threadIdx.x; i < H; i += blockDim.x) o[i] = from_f<act_t>(x[i]);
     return;
@@ -337,13 +337,14 @@ __global__ void add_postnorm_kernel(float* __restrict__ resid, const act_t* __re
   for (int i = threadIdx.x; i < H; i += blockDim.x) {
     const float v = x[i] + mult * (to_f(yr[i]) * inv * w[i]);
     x[i] = v;
-    o[i] = from_f<act_t>(v);
+    if (o != nullptr) o[i] = from_f<act_t>(v);
   }
 }
 
 extern "C" const char* sl_add_postnorm(float* resid, const void* y, const float* w, void* out, int T, int H,
                                        float eps, float mult, hipStream_t stream) {
   SL_CHECK(T >= 0 && H > 0, "add_postnorm: sizes must be positive");
+  SL_CHECK(y != nullptr || out != nullptr, "add_postnorm: nothing to do");
   if (T == 0) return nullptr;
   add_postnorm_kernel<<<T, H >= 2048 ? 512 : 256, 0, stream>>>(resid, (const act_t*)y, w, (act_t*)out, H, eps, mult);
   return sl_launch_status();

@@ -5,11 +5,14 @@
 //                    decay (logsigmoid(z) / tau, or -exp(rate_h) softplus(z)) or plain
 //   short_conv       silu of a causal convolution over time per channel (with or without a bias),
 //                    the last taps - 1 inputs kept in the state slot; heads made unit vectors
+//   stream_conv      the float stream plus a causal convolution over time of itself, as a mixer's
+//                    rows; for one token a sequence also the normed add of the output before it
 //   matrix_scan      the recurrences: decay per key channel (S' = diag(a) S + k v^T), the same
 //                    with the delta rule's correction (u = beta (v - S'^T k)), the matrix
 //                    LSTM (scalar gates with a running maximum, a normaliser n), and the
 //                    state-space form (a scalar decay per head from a step size dt, the input
-//                    times dt, a skip of the token's own input)
+//                    times dt, a skip of the token's own input), and the forget form (S' =
+//                    diag(f) S + (1 - f) v^T, the gate f = l + (1 - l) sigmoid(z) also writes)
 //   head_norm_gate   a head's read-out divided by its root mean square, gain, output gate
 //   projnorm_rope_store  softmax attention's q and k normed over the whole projection, rotated,
 //                    k and v written to their pages
@@ -192,6 +195,130 @@ extern "C" const char* sl_short_conv(const float* buf, int stride, int col, int 
   return sl_launch_status();
 }
 
+// ------------------------------------------------------------------ convolution over the stream
+// out_t = x_t + sum_j w[j] x_(t - taps + 1 + j) per channel of the float stream x, rounded once: what a
+// mixer behind such a convolution reads.  The inputs before a step's first token come from the
+// sequence's slot, as in short_conv_kernel.  Here w lies as [taps][C], so that neighbouring threads
+// read neighbouring values.  VEC consecutive channels a thread.
+template <int VEC> struct __attribute__((aligned(4 * VEC))) conv_vec { float v[VEC]; };
+template <int VEC> struct __attribute__((aligned(sizeof(act_t) * VEC))) conv_act { act_t v[VEC]; };
+
+template <int VEC>
+__global__ __launch_bounds__(256) void stream_conv_kernel(const ShortConv a, act_t* __restrict__ out) {
+  typedef conv_vec<VEC> vec;
+  const int t = blockIdx.x, c = (blockIdx.y * 256 + threadIdx.x) * VEC;
+  if (c >= a.C) return;
+  const int s = a.tok_seq[t];
+  const int first = a.cu_q[s];
+  const int i = t - first, back = a.taps - 1;
+  const bool fresh = a.positions[first] == 0;
+  const float* past = a.state + (size_t)a.slots[s] * a.state_stride + a.state_off;
+  float acc[VEC];
+#pragma unroll
+  for (int u = 0; u < VEC; ++u) acc[u] = 0.f;
+  for (int j = 0; j < a.taps; ++j) {
+    const int idx = i - back + j;
+    if (idx < 0 && fresh) continue;
+    const vec w = *(const vec*)(a.w + (size_t)j * a.C + c);
+    vec x;
+    if (idx >= 0) {
+      x = *(const vec*)(a.buf + (size_t)(first + idx) * a.stride + c);
+    } else {
+#pragma unroll
+      for (int u = 0; u < VEC; ++u) x.v[u] = past[(size_t)(back + idx) * a.C + c + u];
+    }
+#pragma unroll
+    for (int u = 0; u < VEC; ++u) acc[u] += w.v[u] * x.v[u];
+  }
+  const vec x = *(const vec*)(a.buf + (size_t)t * a.stride + c);
+  conv_act<VEC> o;
+#pragma unroll
+  for (int u = 0; u < VEC; ++u) o.v[u] = from_f<act_t>(x.v[u] + acc[u]);
+  *(conv_act<VEC>*)(out + (size_t)t * a.C + c) = o;
+}
+
+// One token a sequence: everything between a sublayer's output and the next mixer's rows in one launch.
+// x += y / sqrt(mean(y^2) + eps) * wy (y == nullptr: x as it is), the convolution over x and the slot's
+// last inputs, and the slot moved on by one.  A block takes a token; a thread's channels are its own
+// throughout, so the slot is read and rewritten without a barrier.  The sums run in the order of the
+// kernels for longer steps.
+constexpr int STREAM_KEEP = 8;
+__global__ void stream_step_kernel(const ShortConv a, float* __restrict__ resid, const act_t* __restrict__ y,
+                                   const float* __restrict__ wy, float eps, int write, act_t* __restrict__ out) {
+  __shared__ float scratch[16];
+  const int t = blockIdx.x, H = a.C, back = a.taps - 1;
+  float* x = resid + (size_t)t * H;
+  const act_t* yr = y != nullptr ? y + (size_t)t * H : nullptr;
+  const int s = a.tok_seq[t];
+  const bool fresh = a.positions[t] == 0;
+  float* keep_in = a.state + (size_t)a.slots[s] * a.state_stride + a.state_off;
+  float inv = 0.f;
+  float yk[STREAM_KEEP];
+  if (yr != nullptr) {
+    float ss = 0.f;
+#pragma unroll
+    for (int u = 0; u < STREAM_KEEP; ++u) {
+      const int c = threadIdx.x + u * blockDim.x;
+      yk[u] = c < H ? to_f(yr[c]) : 0.f;
+      ss += yk[u] * yk[u];
+    }
+    for (int c = threadIdx.x + STREAM_KEEP * blockDim.x; c < H; c += blockDim.x) {
+      const float v = to_f(yr[c]);
+      ss += v * v;
+    }
+    ss = block_sum(ss, scratch);
+    inv = 1.f / sqrtf(ss / (float)H + eps);
+  }
+  auto channel = [&](int c, float yv) {
+    float v = x[c];
+    if (yr != nullptr) {
+      v += yv * inv * wy[c];
+      x[c] = v;
+    }
+    float acc = 0.f;
+    for (int j = 0; j < back; ++j) {
+      const float p = fresh ? 0.f : keep_in[(size_t)j * H + c];
+      if (!fresh) acc += a.w[(size_t)j * H + c] * p;
+      if (write && j > 0) keep_in[(size_t)(j - 1) * H + c] = p;
+    }
+    acc += a.w[(size_t)back * H + c] * v;
+    if (write && back > 0) keep_in[(size_t)(back - 1) * H + c] = v;
+    out[(size_t)t * H + c] = from_f<act_t>(v + acc);
+  };
+#pragma unroll
+  for (int u = 0; u < STREAM_KEEP; ++u) {
+    const int c = threadIdx.x + u * blockDim.x;
+    if (c < H) channel(c, yr != nullptr ? yk[u] : 0.f);
+  }
+  for (int c = threadIdx.x + STREAM_KEEP * blockDim.x; c < H; c += blockDim.x)
+    channel(c, yr != nullptr ? to_f(yr[c]) : 0.f);
+}
+
+// single: every sequence of the step has one token; y (with wy, eps) is taken in that form only.
+extern "C" const char* sl_stream_conv(float* resid, int C, int taps, const float* w, float* state,
+                                      long long state_stride, int state_off, const int* cu_q, const int* positions,
+                                      const int* tok_seq, const int* slots, int S, int T, int write, int single,
+                                      const void* y, const float* wy, float eps, void* out, hipStream_t stream) {
+  SL_CHECK(T >= 0 && S >= 0 && C > 0 && taps >= 1 && taps <= 64, "stream_conv: sizes must be positive, taps <= 64");
+  SL_CHECK(state_off >= 0 && state_off + (long long)(taps - 1) * C <= state_stride,
+           "stream_conv: the last inputs do not fit the state slot");
+  SL_CHECK(!single || S == T, "stream_conv: one token a sequence");
+  SL_CHECK(y == nullptr || (single && wy != nullptr), "stream_conv: a normed output is added for one token a sequence");
+  if (T == 0) return nullptr;
+  const ShortConv a{resid, C, 0, C, taps, w, nullptr, state, state_stride, state_off, cu_q, positions, tok_seq,
+                    slots, 0, 0, 0, 0.f, 1.f, 0, nullptr};
+  if (single) {
+    stream_step_kernel<<<T, C >= 2048 ? 1024 : (C >= 512 ? 512 : 256), 0, stream>>>(a, resid, (const act_t*)y, wy, eps,
+                                                                                 write, (act_t*)out);
+    return sl_launch_status();
+  }
+  const bool whole = C % 4 == 0 && (uintptr_t)resid % 16 == 0 && (uintptr_t)w % 16 == 0 && (uintptr_t)out % 16 == 0;
+  if (whole) stream_conv_kernel<4><<<dim3(T, (C + 1023) / 1024), 256, 0, stream>>>(a, (act_t*)out);
+  else stream_conv_kernel<1><<<dim3(T, (C + 255) / 256), 256, 0, stream>>>(a, (act_t*)out);
+  if (write && taps > 1) short_conv_state_kernel<<<dim3(S, (C + 255) / 256), 256, 0, stream>>>(a, S);
+  return sl_launch_status();
+}
+
 // ------------------------------------------------------------------ the recurrences
 struct MatrixScan {
   const float* src;          // q, k, v of token t at src + t * src_stride + {q,k,v}_col; q and k have G heads
@@ -205,6 +332,7 @@ struct MatrixScan {
   const float* rates;        // state-space, per head: dt = softplus(raw + step_bias[h]), the state keeps
   const float* step_bias;    // exp(-exp(rates[h]) dt) of itself and takes dt k v^T; the read-out adds
   const float* skip;         // skip[h] v
+  const float* lower;        // forget form: [H][D] lower bounds l of the gate; z lies where k lies else
   float cap;
   float* state;              // slot s at state + s * state_stride: S [H][Dv][D]; matrix LSTM: then n [H][D], m [H]
   long long state_stride;
@@ -215,7 +343,7 @@ struct MatrixScan {
   float* out;                // [T][H][Dv]
 };
 
-enum { SCAN_DECAY = 0, SCAN_DELTA = 1, SCAN_LSTM = 2, SCAN_SSD = 3 };
+enum { SCAN_DECAY = 0, SCAN_DELTA = 1, SCAN_LSTM = 2, SCAN_SSD = 3, SCAN_FORGET = 4 };
 constexpr int SCAN_ROWS = 8;      // key channels a lane owns: channels 8 p .. 8 p + 7
 
 // Sum over the P lanes that share a column (P a power of two, the lanes adjacent and aligned); every
@@ -281,6 +409,15 @@ __global__ __launch_bounds__(512) void matrix_scan_kernel(const MatrixScan a, in
     // chunk before: at most 8 values of q, k and the decays and 8 of v a thread (the host keeps CH
     // within that).
     float pq[8], pk[8], pd[8], pv[8], g0 = 0.f, g1 = 0.f;
+    // forget form: the bound of the key channel that place e of this thread holds in every chunk
+    float bound[8];
+    if (MODE == SCAN_FORGET) {
+#pragma unroll
+      for (int e = 0; e < 8; ++e) {
+        const int r = (tid + e * 256) & (Dp - 1);
+        bound[e] = r < a.D ? a.lower[h * a.D + r] : 0.f;
+      }
+    }
     auto ask = [&](int t0, int nt) {
 #pragma unroll
       for (int e = 0; e < 8; ++e) {
@@ -293,9 +430,9 @@ __global__ __launch_bounds__(512) void matrix_scan_kernel(const MatrixScan a, in
           const int tt = idx >> lgDp, r = idx & (Dp - 1);          // (Dp and cols are powers of two)
           const size_t t = t0 + tt;
           if (r < a.D) {
-            pq[e] = a.src[t * a.src_stride + a.q_col + g * a.D + r] * a.q_scale;
+            pq[e] = a.src[t * a.src_stride + a.q_col + g * a.D + r] * (MODE == SCAN_FORGET ? 1.f : a.q_scale);
             pk[e] = a.src[t * a.src_stride + a.k_col + g * a.D + r];
-            if (!SCALAR) pd[e] = a.log_decay[(t * a.H + h) * a.D + r];
+            if (!SCALAR && MODE != SCAN_FORGET) pd[e] = a.log_decay[(t * a.H + h) * a.D + r];
           }
         }
         if (idx < nt * cols) {
@@ -304,7 +441,7 @@ __global__ __launch_bounds__(512) void matrix_scan_kernel(const MatrixScan a, in
           else if (cc < a.Dv) pv[e] = a.src[(size_t)(t0 + tt) * a.src_stride + a.v_col + h * a.Dv + cc];
         }
       }
-      if (MODE != SCAN_DECAY && tid < 64 && tid < nt) {
+      if (MODE != SCAN_DECAY && MODE != SCAN_FORGET && tid < 64 && tid < nt) {
         const float* gr = a.gates + (size_t)(t0 + tid) * a.gate_stride;
         g0 = gr[a.i_col + h];
         if (MODE == SCAN_LSTM) g1 = gr[a.f_col + h];
@@ -338,9 +475,19 @@ __global__ __launch_bounds__(512) void matrix_scan_kernel(const MatrixScan a, in
             // the lanes of a column read together are then side by side and take every LDS bank once
             const int r = idx & (Dp - 1);
             const int at = (idx - r) + ((r & (ROWS - 1)) >> 2) * 4 * P + (r / ROWS) * 4 + (r & 3);
-            base[oq + at] = pq[e];
-            base[ok + at] = pk[e];
-            if (!SCALAR) base[oa + at] = expf(pd[e]);
+            if (MODE == SCAN_FORGET) {
+              // f = l + (1 - l) sigmoid(z) and 1 - f = (1 - l) sigmoid(-z), each from its own side: no
+              // difference of nearly equal numbers where the gate is almost open; q passes silu
+              const float en = expf(-fabsf(pk[e])), big = 1.f / (1.f + en), small = en * big;
+              const bool pos = pk[e] >= 0.f, in = r < a.D;
+              base[oq + at] = pq[e] * sigmoidf_(pq[e]) * a.q_scale;
+              base[ok + at] = in ? (1.f - bound[e]) * (pos ? small : big) : 0.f;
+              base[oa + at] = in ? bound[e] + (1.f - bound[e]) * (pos ? big : small) : 1.f;
+            } else {
+              base[oq + at] = pq[e];
+              base[ok + at] = pk[e];
+              if (!SCALAR) base[oa + at] = expf(pd[e]);
+            }
           }
           if (idx < nt * cols) base[ov + idx] = pv[e];
         }
@@ -436,7 +583,7 @@ __global__ __launch_bounds__(512) void matrix_scan_kernel(const MatrixScan a, in
       }
       const float v = sv[tt * cols + cl];
       float part[ROWS];
-      if (MODE == SCAN_DECAY) {
+      if (MODE == SCAN_DECAY || MODE == SCAN_FORGET) {
 #pragma unroll
         for (int i = 0; i < ROWS; ++i) {
           S[i] = d[i] * S[i] + k[i] * v;
@@ -493,17 +640,19 @@ __global__ __launch_bounds__(512) void matrix_scan_kernel(const MatrixScan a, in
 extern "C" const char* sl_matrix_scan(int mode, const float* src, int src_stride, int q_col, int k_col, int v_col,
                                       int H, int G, int D, int Dv, const float* log_decay, float q_scale,
                                       const float* gates, int gate_stride, int i_col, int f_col, float cap,
-                                      const float* rates, const float* step_bias, const float* skip, float* state, long long state_stride, const int* cu_q, const int* positions,
+                                      const float* rates, const float* step_bias, const float* skip, const float* lower, float* state, long long state_stride,
+                                      const int* cu_q, const int* positions,
                                       const int* slots, int S, int T, int write, float* out, hipStream_t stream) {
-  SL_CHECK(mode >= 0 && mode <= 3, "matrix_scan: unknown mode");
+  SL_CHECK(mode >= 0 && mode <= 4, "matrix_scan: unknown mode");
   SL_CHECK(S >= 0 && T >= 0 && H > 0 && G > 0 && H % G == 0 && Dv > 0, "matrix_scan: sizes must be positive");
   SL_CHECK(D >= 1 && D <= 64 * SCAN_ROWS, "matrix_scan: at most 512 key channels a head");
   SL_CHECK(q_col >= 0 && k_col >= 0 && v_col >= 0 && q_col + G * D <= src_stride && k_col + G * D <= src_stride &&
            v_col + H * Dv <= src_stride, "matrix_scan: q, k or v do not fit the rows");
-  SL_CHECK(mode == SCAN_LSTM || mode == SCAN_SSD || log_decay != nullptr, "matrix_scan: decays are missing");
+  SL_CHECK(mode == SCAN_LSTM || mode == SCAN_SSD || mode == SCAN_FORGET || log_decay != nullptr, "matrix_scan: decays are missing");
+  SL_CHECK(mode != SCAN_FORGET || (lower != nullptr && G == H), "matrix_scan: the forget form needs a bound per channel, and its gates per head");
   SL_CHECK(mode != SCAN_SSD || (rates != nullptr && step_bias != nullptr && skip != nullptr),
            "matrix_scan: the state-space form needs rates, step biases and skips per head");
-  SL_CHECK(mode == SCAN_DECAY || (gates != nullptr && i_col >= 0 && i_col + H <= gate_stride),
+  SL_CHECK(mode == SCAN_DECAY || mode == SCAN_FORGET || (gates != nullptr && i_col >= 0 && i_col + H <= gate_stride),
            "matrix_scan: gates are missing or do not fit their rows");
   SL_CHECK(mode != SCAN_LSTM || (f_col >= 0 && f_col + H <= gate_stride && cap > 0.f),
            "matrix_scan: the forget gates do not fit their rows");
@@ -520,18 +669,20 @@ extern "C" const char* sl_matrix_scan(int mode, const float* src, int src_stride
   const bool scalar = mode == SCAN_LSTM || mode == SCAN_SSD;
   const size_t lds = 2 * (size_t)CH * ((scalar ? 2 : 3) * Dp + 2 * cols + 4) * sizeof(float);   // two halves
   const MatrixScan a{src, src_stride, q_col, k_col, v_col, H, G, D, Dv, log_decay, q_scale, gates, gate_stride,
-                     i_col, f_col, rates, step_bias, skip, cap, state, state_stride, cu_q, positions, slots, write, out};
+                     i_col, f_col, rates, step_bias, skip, lower, cap, state, state_stride, cu_q, positions, slots, write, out};
   const int vcols = mode == SCAN_LSTM ? cols - 1 : cols;       // (the matrix LSTM's last column group carries n)
   const dim3 grid(S, H, (Dv + vcols - 1) / vcols);
   if (mode == SCAN_DECAY) matrix_scan_kernel<SCAN_DECAY, SCAN_ROWS><<<grid, 512, lds, stream>>>(a, P, CH);
   else if (mode == SCAN_DELTA) matrix_scan_kernel<SCAN_DELTA, SCAN_ROWS><<<grid, 512, lds, stream>>>(a, P, CH);
   else if (mode == SCAN_SSD) matrix_scan_kernel<SCAN_SSD, SCAN_ROWS><<<grid, 512, lds, stream>>>(a, P, CH);
+  else if (mode == SCAN_FORGET) matrix_scan_kernel<SCAN_FORGET, SCAN_ROWS><<<grid, 512, lds, stream>>>(a, P, CH);
   else matrix_scan_kernel<SCAN_LSTM, SCAN_ROWS><<<grid, 512, lds, stream>>>(a, P, CH);
   return sl_launch_status();
 }
 
 // ------------------------------------------------------------------ read-out: norm, gain, gate
-// One wavefront per (token, head): o / sqrt(mean(o^2) + eps) * w * act(gate); act 0: sigmoid, 1: silu.
+// One wavefront per (token, head): o / sqrt(mean(o^2) + eps) * w * act(gate); act 0: sigmoid, 1: silu;
+// no gate (nullptr): the norm alone.
 // gate_first: the gate comes before the norm, x = o * act(gate), then x / sqrt(mean(x^2) + eps) * w.
 __global__ __launch_bounds__(64) void head_norm_gate_kernel(const float* __restrict__ o, int H, int Dv,
                                                             const float* __restrict__ w, int per_head, float eps,
@@ -541,12 +692,12 @@ __global__ __launch_bounds__(64) void head_norm_gate_kernel(const float* __restr
   const size_t t = blockIdx.x;
   const int h = blockIdx.y, lane = threadIdx.x;
   const float* x = o + (t * H + h) * Dv;
-  const float* gr = gate + t * gate_stride + gate_col + h * Dv;
+  const float* gr = gate != nullptr ? gate + t * gate_stride + gate_col + h * Dv : nullptr;
   const float* wr = w + (per_head ? h * Dv : 0);
   float ss = 0.f;
   for (int d = lane; d < Dv; d += 64) {
     float v = x[d];
-    if (gate_first) {
+    if (gate_first && gr != nullptr) {
       const float z = gr[d];
       v *= act == 0 ? sigmoidf_(z) : z * sigmoidf_(z);
     }
@@ -554,6 +705,10 @@ __global__ __launch_bounds__(64) void head_norm_gate_kernel(const float* __restr
   }
   const float inv = 1.f / sqrtf(wave_sum(ss) / (float)Dv + eps);
   for (int d = lane; d < Dv; d += 64) {
+    if (gr == nullptr) {
+      out[(t * H + h) * Dv + d] = from_f<act_t>(x[d] * inv * wr[d]);
+      continue;
+    }
     const float z = gr[d];
     const float gv = act == 0 ? sigmoidf_(z) : z * sigmoidf_(z);
     out[(t * H + h) * Dv + d] = from_f<act_t>(gate_first ? (x[d] * gv) * inv * wr[d] : x[d] * inv * wr[d] * gv);
@@ -564,7 +719,7 @@ extern "C" const char* sl_head_norm_gate(const float* o, int T, int H, int Dv, c
                                          float eps, const float* gate, int gate_stride, int gate_col, int act,
                                          int gate_first, void* out, hipStream_t stream) {
   SL_CHECK(T >= 0 && H > 0 && Dv > 0, "head_norm_gate: sizes must be positive");
-  SL_CHECK(gate_col >= 0 && gate_col + H * Dv <= gate_stride, "head_norm_gate: the gates do not fit their rows");
+  SL_CHECK(gate == nullptr || (gate_col >= 0 && gate_col + H * Dv <= gate_stride), "head_norm_gate: the gates do not fit their rows");
   SL_CHECK(act == 0 || act == 1, "head_norm_gate: the gate is sigmoid (0) or silu (1)");
   if (T == 0) return nullptr;
   head_norm_gate_kernel<<<dim3(T, H), 64, 0, stream>>>(o, H, Dv, w, per_head, eps, gate, gate_stride, gate_col,
@@ -651,12 +806,15 @@ __global__ void projnorm_rope_store_kernel(const float* __restrict__ buf, int st
       vc[((pg * G + e / Dv) * Dv + e % Dv) * page + off] = from_f<act_t>(row[v_col + e]);
 }
 
-// The same without a norm over the projection, where nothing ties a token's heads together: one
-// wavefront per (token, head of q, k or v), so that a step of few tokens still fills the chip
+// The same without a norm over the projection, where nothing ties a token's heads together (no norm, or
+// one per head: qw [H][D] and kw [G][D] are then the gains of a head divided by its own root mean square):
+// one wavefront per (token, head of q, k or v), so that a step of few tokens still fills the chip
 // and the convolution's loads (a head's channels over the taps, and their partners' for the
 // rotation) are all in flight together.  The sums run in the order of the kernel above.
 __global__ __launch_bounds__(64) void rope_store_heads_kernel(const float* __restrict__ buf, int stride, int H, int G, int D,
-                                                              int Dv, int rot, const float* __restrict__ cosv,
+                                                              int Dv, const float* __restrict__ qw,
+                                                              const float* __restrict__ kw, float eps, int rot,
+                                                              const float* __restrict__ cosv,
                                                               const float* __restrict__ sinv,
                                                               const int* __restrict__ slots, act_t* __restrict__ kc,
                                                               act_t* __restrict__ vc, int page,
@@ -700,11 +858,23 @@ __global__ __launch_bounds__(64) void rope_store_heads_kernel(const float* __res
   if (!is_q && slots == nullptr) return;
   const int base = hb * D;                             // (k heads follow the q heads in the row)
   const int half = rot / 2;
+  const float* gain = qw == nullptr ? nullptr : (is_q ? qw + base : kw + (hb - H) * D);
+  float inv = 1.f;
+  if (gain != nullptr) {
+    float ss = 0.f;
+    for (int d = lane; d < D; d += 64) {
+      const float v = value(base + d);
+      ss += v * v;
+    }
+    inv = 1.f / sqrtf(wave_sum(ss) / (float)D + eps);
+  }
   for (int d = lane; d < D; d += 64) {
     float v = value(base + d);
+    if (gain != nullptr) v = v * inv * gain[d];
     if (d < rot) {
-      const int p = d < half ? d : d - half;
-      const float o = value(base + (d < half ? d + half : d - half));
+      const int p = d < half ? d : d - half, pd = d < half ? d + half : d - half;
+      float o = value(base + pd);
+      if (gain != nullptr) o = o * inv * gain[pd];
       const float cs = cosv[t * half + p], sn = sinv[t * half + p];
       v = d < half ? v * cs - o * sn : v * cs + o * sn;
     }
@@ -714,7 +884,7 @@ __global__ __launch_bounds__(64) void rope_store_heads_kernel(const float* __res
 }
 
 extern "C" const char* sl_projnorm_rope_store(const float* buf, int stride, int T, int H, int G, int D, int Dv,
-                                              const float* qw, const float* kw, float eps, int rot,
+                                              const float* qw, const float* kw, float eps, int per_head, int rot,
                                               const float* cosv, const float* sinv, const int* slots, void* kc,
                                               void* vc, int page, void* q_out, int v_col,
                                               const float* taps_w, int taps, int conv_C, float* state,
@@ -746,8 +916,10 @@ extern "C" const char* sl_projnorm_rope_store(const float* buf, int stride, int 
   // (few tokens: a wavefront per head fills the chip; many: a block per token computes every channel's
   // convolution once, where the heads' wavefronts compute the rotated ones twice: 2,048 tokens of 20 heads
   // of 128 channels, 4 taps: 32 against 50 us; 8 tokens: 28 against 9 us)
-  if (qw == nullptr && H + 2 * G <= 65535 && T < 512)
-    rope_store_heads_kernel<<<dim3(T, H + 2 * G), 64, 0, stream>>>(buf, stride, H, G, D, Dv, rot, cosv, sinv, slots,
+  // (a norm per head always runs there: a wavefront has the whole head)
+  SL_CHECK(!per_head || H + 2 * G <= 65535, "projnorm_rope_store: too many heads");
+  if ((qw != nullptr && per_head) || (qw == nullptr && H + 2 * G <= 65535 && T < 512))
+    rope_store_heads_kernel<<<dim3(T, H + 2 * G), 64, 0, stream>>>(buf, stride, H, G, D, Dv, qw, kw, eps, rot, cosv, sinv, slots,
                                                                    (act_t*)kc, (act_t*)vc, page, (act_t*)q_out, v_col, cv);
   else   // (a step of few tokens has few blocks: wider ones shorten each block's loops over the row)
     projnorm_rope_store_kernel<<<T, T <= 64 ? 1024 : 256, lds, stream>>>(buf, stride, H, G, D, Dv, qw, kw, eps, rot, cosv, sinv, slots,

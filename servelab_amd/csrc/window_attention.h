@@ -22,6 +22,8 @@ struct WindowAttention {
   const float* sinks;        // [nh] or nullptr
   const act_t* gate;         // gate of (t, h) at gate[t * gate_stride + h], or nullptr
   int gate_stride;
+  const float* channel_gate; // gate of (t, h, d) at channel_gate[t * channel_stride + h * Dv + d], or nullptr
+  int channel_stride;
   act_t* out;                // [tokens][nh][Dv]
   int nsplit;
   float* part_o;             // [tokens][nh][nsplit][Dv]
@@ -36,7 +38,7 @@ __device__ __forceinline__ float sigmoidf_(float x) { return 1.f / (1.f + expf(-
 __global__ __launch_bounds__(64) void window_attention_combine_kernel(
     const float* __restrict__ part_o, const float* __restrict__ part_ml, int nsplit, int nh, int Dv,
     const float* __restrict__ sinks, const act_t* __restrict__ gate, int gate_stride,
-    act_t* __restrict__ out) {
+    const float* __restrict__ channel_gate, int channel_stride, act_t* __restrict__ out) {
   __shared__ float ws[64];
   const int t = blockIdx.x, h = blockIdx.y, lane = threadIdx.x;
   const size_t base = ((size_t)t * nh + h) * nsplit;
@@ -65,6 +67,7 @@ __global__ __launch_bounds__(64) void window_attention_combine_kernel(
 #pragma unroll
       for (int u = 0; u < 8; ++u) s += (j + u < nsplit ? ws[j + u] : 0.f) * v[u];
     }
+    if (channel_gate != nullptr) s *= sigmoidf_(channel_gate[(size_t)t * channel_stride + h * Dv + d]);
     o[d] = from_f<act_t>(s * f);
   }
 }

@@ -9,7 +9,8 @@
 //   * a distance bias: slope_h * (i - j) is taken off the scaled score;
 //   * a sink: exp(sink_h) enters the softmax's denominator once, without a key
 //     or a value;
-//   * an output gate: the head's output is multiplied by sigmoid(gate[t, h]).
+//   * an output gate: the head's output is multiplied by sigmoid(gate[t, h]), or
+//     channel by channel by sigmoid(channel_gate[t, h, d]) (float rows).
 // Scores, weights, the running maximum and sum and the output sums are float
 // in both builds; q, keys and values arrive in the activation type.
 //
@@ -184,9 +185,12 @@ __global__ __launch_bounds__(WA_THREADS) void window_attention_kernel(const Wind
   float f = w / (l * w + extra);
   if (a.gate != nullptr) f *= sigmoidf_(to_f(a.gate[(size_t)(q0 + tok) * a.gate_stride + head]));
   act_t* o = a.out + row * Dv;
+  const float* cg = a.channel_gate != nullptr
+      ? a.channel_gate + (size_t)(q0 + tok) * a.channel_stride + (size_t)head * Dv : nullptr;
 #pragma unroll
   for (int j = 0; j < NJ; ++j)
-    if (16 * j + sub < Dv) o[16 * j + sub] = from_f<act_t>(acc[j] * f);
+    if (16 * j + sub < Dv)
+      o[16 * j + sub] = from_f<act_t>(acc[j] * (cg != nullptr ? f * sigmoidf_(cg[16 * j + sub]) : f));
 }
 
 template <int KB>
@@ -216,8 +220,8 @@ extern "C" const char* sl_window_attention(
     const void* q, int q_stride, const void* kc, const void* vc, const int* tables, int max_pages,
     const int* cu_q, const int* positions, int num_seqs, int max_q_len, int num_tokens, int nh,
     int nkv, int Dk, int Dv, int page, float scale, float softcap, int window, int keep_first, const float* slopes,
-    const float* sinks, const void* gate, int gate_stride, void* out, int nsplit, float* part_o,
-    float* part_ml, hipStream_t stream) {
+    const float* sinks, const void* gate, int gate_stride, const float* channel_gate, int channel_stride, void* out,
+    int nsplit, float* part_o, float* part_ml, hipStream_t stream) {
   SL_CHECK(num_seqs >= 0 && max_q_len >= 1 && nh > 0 && nkv > 0 && nh % nkv == 0,
            "window attention: heads must be a positive multiple of kv heads");
   SL_CHECK(Dk > 0 && Dv > 0 && Dv <= 512, "window attention: value width must be in 1..512");
@@ -229,13 +233,15 @@ extern "C" const char* sl_window_attention(
   SL_CHECK(nsplit == 1 || (part_o != nullptr && part_ml != nullptr),
            "window attention: shares of the keys need the partial buffers");
   SL_CHECK(gate == nullptr || gate_stride >= nh, "window attention: gate rows are shorter than the heads");
+  SL_CHECK(channel_gate == nullptr || channel_stride >= nh * Dv, "window attention: gate rows are shorter than the output");
   if (num_seqs == 0 || num_tokens == 0) return nullptr;
   const long long cols = (long long)max_q_len * (nh / nkv);
   const long long tiles = (cols + WA_COLS - 1) / WA_COLS;
   SL_CHECK(tiles * nsplit <= 1 << 30, "window attention: too many column tiles");
   const WindowAttention a{(const act_t*)q, q_stride, (const act_t*)kc, (const act_t*)vc, tables, max_pages,
                           cu_q, positions, nh, nkv, Dk, Dv, page, scale, softcap, window, keep_first, slopes, sinks,
-                          (const act_t*)gate, gate_stride, (act_t*)out, nsplit, part_o, part_ml};
+                          (const act_t*)gate, gate_stride, channel_gate, channel_stride, (act_t*)out, nsplit, part_o,
+                          part_ml};
   const dim3 grid((unsigned)(tiles * nsplit), nkv, num_seqs);
   const int DkP = (Dk + 3) & ~3;
   auto need = [&](int KB) {
@@ -250,7 +256,8 @@ extern "C" const char* sl_window_attention(
   }
   if (e || nsplit == 1) return e;
   window_attention_combine_kernel<<<dim3(num_tokens, nh, (Dv + 63) / 64), 64, 0, stream>>>(
-      part_o, part_ml, nsplit, nh, Dv, sinks, (const act_t*)gate, gate_stride, (act_t*)out);
+      part_o, part_ml, nsplit, nh, Dv, sinks, (const act_t*)gate, gate_stride, channel_gate, channel_stride,
+      (act_t*)out);
   return sl_launch_status();
 }
 

@@ -356,9 +356,17 @@ __global__ __launch_bounds__(THREADS) void window_attention_mfma_kernel(const Wi
   float f = w / (l * w + extra);
   if (a.gate != nullptr) f *= sigmoidf_(to_f(a.gate[(size_t)(q0 + tok) * a.gate_stride + head]));
   __bf16* op = a.out + row * DV + 4 * gq;
+  const float* cg = a.channel_gate != nullptr
+      ? a.channel_gate + (size_t)(q0 + tok) * a.channel_stride + (size_t)head * DV + 4 * gq : nullptr;
 #pragma unroll
   for (int dd = 0; dd < DD; ++dd) {
     bf16x4 r;
+    if (cg != nullptr) {
+      struct __attribute__((aligned(4))) gates4 { float v[4]; };      // (one load, whatever the rows' alignment)
+      const gates4 z = *(const gates4*)(cg + 16 * dd);
+#pragma unroll
+      for (int e = 0; e < 4; ++e) o[dd][e] *= sigmoidf_(z.v[e]);
+    }
 #pragma unroll
     for (int e = 0; e < 4; ++e) r[e] = (__bf16)(o[dd][e] * f);
     *(bf16x4*)(op + 16 * dd) = r;
@@ -386,8 +394,8 @@ extern "C" const char* sl_window_attention_mfma(
     const void* q, int q_stride, const void* kc, const void* vc, const int* tables, int max_pages,
     const int* cu_q, const int* positions, int num_seqs, int max_q_len, int num_tokens, int nh,
     int nkv, int Dk, int Dv, int page, float scale, float softcap, int window, int keep_first, const float* slopes,
-    const float* sinks, const void* gate, int gate_stride, void* out, int nsplit, float* part_o,
-    float* part_ml, hipStream_t stream) {
+    const float* sinks, const void* gate, int gate_stride, const float* channel_gate, int channel_stride, void* out,
+    int nsplit, float* part_o, float* part_ml, hipStream_t stream) {
   SL_CHECK(Dk == DK && Dv == DV && (vc == nullptr) == VK, "window attention (matrix cores): built for other widths");
   SL_CHECK(num_seqs >= 0 && max_q_len >= 1 && nh > 0 && nkv > 0 && nh % nkv == 0,
            "window attention: heads must be a positive multiple of kv heads");
@@ -398,13 +406,15 @@ extern "C" const char* sl_window_attention_mfma(
   SL_CHECK(nsplit == 1 || (part_o != nullptr && part_ml != nullptr),
            "window attention: shares of the keys need the partial buffers");
   SL_CHECK(gate == nullptr || gate_stride >= nh, "window attention: gate rows are shorter than the heads");
+  SL_CHECK(channel_gate == nullptr || channel_stride >= nh * Dv, "window attention: gate rows are shorter than the output");
   SL_CHECK((uintptr_t)q % 16 == 0 && q_stride % 8 == 0 && (uintptr_t)kc % 16 == 0 && (uintptr_t)vc % 16 == 0 &&
            (uintptr_t)out % 8 == 0 && (uintptr_t)part_o % 16 == 0,
            "window attention (matrix cores): operands must be 16-byte aligned");
   if (num_seqs == 0 || num_tokens == 0) return nullptr;
   const WindowAttention a{(const act_t*)q, q_stride, (const act_t*)kc, (const act_t*)vc, tables, max_pages,
                           cu_q, positions, nh, nkv, Dk, Dv, page, scale, softcap, window, keep_first, slopes, sinks,
-                          (const act_t*)gate, gate_stride, (act_t*)out, nsplit, part_o, part_ml};
+                          (const act_t*)gate, gate_stride, channel_gate, channel_stride, (act_t*)out, nsplit, part_o,
+                          part_ml};
   const long long cols = (long long)max_q_len * (nh / nkv);
   const long long tiles = (cols + COLS - 1) / COLS;
   SL_CHECK(tiles * nsplit <= 1 << 30, "window attention: too many column tiles");
@@ -412,6 +422,7 @@ extern "C" const char* sl_window_attention_mfma(
   const char* e = launch_mfma(a, grid, stream);
   if (e || nsplit == 1) return e;
   window_attention_combine_kernel<<<dim3(num_tokens, nh, (Dv + 63) / 64), 64, 0, stream>>>(
-      part_o, part_ml, nsplit, nh, Dv, sinks, (const act_t*)gate, gate_stride, (act_t*)out);
+      part_o, part_ml, nsplit, nh, Dv, sinks, (const act_t*)gate, gate_stride, channel_gate, channel_stride,
+      (act_t*)out);
   return sl_launch_status();
 }

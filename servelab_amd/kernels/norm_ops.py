@@ -10,14 +10,20 @@ from .values import (Deferred, KernelError, PartialSums, ScaledRows, TiledRows, 
 
 class NormOps:
     # ------------------------------------------------------------ embedding
-    def embed(self, ids, table, scale=1.0):
-        """The rows of ``table`` at ``ids`` times ``scale``, as the float32 stream [T, H]."""
+    def embed(self, ids, table, scale=1.0, positions=None, pos_table=None):
+        """The rows of ``table`` at ``ids`` times ``scale``, as the float32 stream [T, H]; with
+        ``pos_table`` [P, H] the rows at ``positions`` (int32, each below P) are added, unscaled."""
         T = ids.shape[0]
         V, H = table.shape
         self._check(ids, torch.int32, (T,), "ids")
         self._check(table, self.act_dtype, None, "embedding table")
         out = self._new((T, H), torch.float32)
-        self._call("elementwise", "sl_embed", _p(ids), _p(table), _p(out), T, H, V, _c_float(scale))
+        if pos_table is not None:
+            self._check(positions, torch.int32, (T,), "positions")
+            self._check(pos_table, self.act_dtype, (pos_table.shape[0], H), "position table")
+        self._call("elementwise", "sl_embed", _p(ids), _p(table), _p(out), T, H, V, _c_float(scale),
+                   _p(positions) if pos_table is not None else None, _p(pos_table),
+                   pos_table.shape[0] if pos_table is not None else 0)
         return out
 
     def stream_pair(self, resid, delta, other):

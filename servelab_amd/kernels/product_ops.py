@@ -33,7 +33,7 @@ class ProductOps:
         return two < 0.97 * one
 
     def _skinny(self, x, weight, bias, y, M, N, K, out_f32=False, gated=False, scaled=None,
-                resid=None, next_gain=None, out_parts=None, rope=None, y_tiled=False):
+                resid=None, next_gain=None, out_parts=None, rope=None, y_tiled=False, act=0):
         """One call of the few-rows kernel (at most 16 rows) in any of its forms."""
         parts = scaled.parts if scaled is not None else None
         x_tiled = scaled.tiled if scaled is not None else 0
@@ -47,7 +47,8 @@ class ProductOps:
                    _c_float(scaled.eps if scaled is not None else 0.0),
                    _p(scaled.rows) if scaled is not None else None, _p(resid), _p(next_gain),
                    _p(out_parts), ctypes.byref(rope) if rope is not None else None,
-                   int(pair), int(x_tiled), int(y_tiled), th, int(M <= 8 and not pair and self.PAIR_X_LOADS))
+                   int(pair), int(x_tiled), int(y_tiled), th, int(M <= 8 and not pair and self.PAIR_X_LOADS),
+                   int(act))
 
     # --------------------------------------------------------------- linear
     def plan_weights(self, total_bytes: int) -> str:
@@ -228,14 +229,14 @@ class ProductOps:
             return self.linear_tiled(x, w, bias, out_f32)
         return self.linear_library(x, w, bias)
 
-    def linear_wide(self, x, weight, bias, out_f32=False, gated=False):
+    def linear_wide(self, x, weight, bias, out_f32=False, gated=False, act=0):
         M, K = x.shape
         N = weight.shape[0]
         if weight.tiled is None:
             raise KernelError("linear_wide needs the tiled copy of the weight")
         y = self._new((M, N // 2 if gated else N), torch.float32 if out_f32 else None)
         self._call("gemm", "sl_gemm_wide", _p(x), _p(weight.tiled), _p(bias), _p(y), M, N, K,
-                   int(out_f32), int(gated))
+                   int(out_f32), int(gated), int(act))
         return y
 
     def _takes_mid(self, M, N, K) -> bool:
@@ -256,7 +257,7 @@ class ProductOps:
         return self.SKINNY_MAX_M
 
     def linear_mid(self, x, weight, bias, out_f32=False, gated=False, ks=None, partial=False,
-                   target=None):
+                   target=None, act=0):
         """17..128 rows with x staged through LDS; K split over workgroups when
         N alone gives too few of them.  ``partial``: a split product comes back
         as ``PartialSums`` for its reader to add up."""
@@ -268,15 +269,15 @@ class ProductOps:
         if ks is None:
             if target is None:
                 target = self.MID_PARTIAL_WORKGROUPS if partial else self.MID_TARGET_WORKGROUPS
-            ks = 1 if gated else max(1, min(16, K // 32 // 4, -(-target // wgs)))
+            ks = 1 if gated or act else max(1, min(16, K // 32 // 4, -(-target // wgs)))
         part = self._new((ks, M, N), torch.float32) if ks > 1 else None
         if partial and ks > 1:
             self._call("gemm", "sl_gemm_mid", _p(x), _p(weight.tiled), None, None, M, N, K,
-                       0, 0, int(ks), self.MID_WIDE_WORKGROUPS, self._num_cus, _p(part))
+                       0, 0, int(ks), self.MID_WIDE_WORKGROUPS, self._num_cus, _p(part), 0)
             return PartialSums(part, bias)
         y = self._new((M, N // 2 if gated else N), torch.float32 if out_f32 else None)
         self._call("gemm", "sl_gemm_mid", _p(x), _p(weight.tiled), _p(bias), _p(y), M, N, K,
-                   int(out_f32), int(gated), int(ks), self.MID_WIDE_WORKGROUPS, self._num_cus, _p(part))
+                   int(out_f32), int(gated), int(ks), self.MID_WIDE_WORKGROUPS, self._num_cus, _p(part), int(act))
         return y
 
     def _block_plan(self, M, N, K, weight):
@@ -441,6 +442,45 @@ class ProductOps:
                  and w_down.tiled is not None and w_down.shape[1] == inner and w_gate_up.shape[0] % 16 == 0)
         h = self.gated_linear(x, w_gate_up, block, _tiled_out=tiled, activation=activation, bias=bias_gate_up)
         return self.linear(h, w_down, bias_down, defer=defer)
+
+    def activated_linear(self, x, weight, activation, bias=None, _tiled_out=False):
+        """act(x W^T + b) for an ``activation`` of ``activate``.  Few rows and a tiled weight: the
+        activation sits in the product's epilogue, on its float32 sums."""
+        if not isinstance(weight, LinearWeight):
+            weight = LinearWeight(weight)
+        code = activation_code(activation, ("silu", "relu", "relu2", "gelu_tanh"))
+        if isinstance(x, ScaledRows):
+            x = self.finish_scaled_rows(x)
+        M, K = x.shape
+        N = weight.shape[0]
+        if M > self._few_rows_limit(weight) or M == 0:
+            return self.activate(self.linear(x, weight, bias), activation)
+        self._check(x, self.act_dtype, None, "x")
+        if weight.shape != (N, K):
+            raise KernelError(f"weight has shape {list(weight.shape)}, x has {K} columns")
+        if bias is not None:
+            self._check(bias, torch.float32, (N,), "bias")
+        if M >= self._wide_from(min(N, K)):
+            if self._takes_mid(M, N, K):
+                return self.linear_mid(x, weight, bias, act=code)
+            return self.linear_wide(x, weight, bias, act=code)
+        y = self._new((M, N))
+        self._skinny(x, weight, bias, y, M, N, K, act=code, y_tiled=_tiled_out)
+        return TiledRows(y, (M, N)) if _tiled_out else y
+
+    def plain_mlp(self, x, w_up, w_down, activation, defer=False):
+        """down(act(up x)) without a gate and without biases; with few rows what lies between the two
+        products is kept in the layout the second one reads best (rows by k-step)."""
+        if not isinstance(w_up, LinearWeight):
+            w_up = LinearWeight(w_up)
+        if not isinstance(w_down, LinearWeight):
+            w_down = LinearWeight(w_down)
+        M, inner = x.shape[0], w_up.shape[0]
+        tiled = (self.act_dtype == torch.bfloat16 and self.tile_few_rows and 1 < M <= self._fused_rows(w_down.shape[0])
+                 and M < self._wide_from(min(w_up.shape)) and inner % 32 == 0 and w_up.tiled is not None
+                 and w_down.tiled is not None and w_down.shape[1] == inner)
+        h = self.activated_linear(x, w_up, activation, _tiled_out=tiled)
+        return self.linear(h, w_down, None, defer=defer)
 
     def linear_rows(self, x, w, bias, out_f32=False):
         M, K = x.shape

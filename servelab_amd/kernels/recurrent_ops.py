@@ -16,7 +16,7 @@ from .values import KernelError, _c_float, _p, activation_code
 _ll = ctypes.c_longlong
 
 _EXPAND_MODES = {"plain": 0, "log_sigmoid": 1, "rate_softplus": 2}
-_SCAN_DECAY, _SCAN_DELTA, _SCAN_LSTM, _SCAN_SSD = 0, 1, 2, 3
+_SCAN_DECAY, _SCAN_DELTA, _SCAN_LSTM, _SCAN_SSD, _SCAN_FORGET = 0, 1, 2, 3, 4
 _TILE_ROWS = (16, 64, 128)    # rows of a row tile of the grouped products (routed.hip)
 
 
@@ -47,15 +47,15 @@ class RecurrentOps:
     ROUTED_WIDE_TILE_ROWS = 48    # rows an expert has on average from which row tiles hold 64 rows
 
     # ------------------------------------------------- norm on an output
-    def add_postnorm(self, resid, y, weight, eps, mult):
+    def add_postnorm(self, resid, y, weight, eps, mult, want_rows=True):
         """resid += mult * y / sqrt(mean(y^2) + eps) * weight in place (float32); returns the
-        stream's rows in the activation dtype.  ``y`` None: only those rows."""
+        stream's rows in the activation dtype (``want_rows`` False: None).  ``y`` None: only those rows."""
         T, H = resid.shape
         self._check(resid, torch.float32, None, "residual stream")
         self._check(weight, torch.float32, (H,), "norm weight")
         if y is not None:
             self._check(y, self.act_dtype, (T, H), "sublayer output")
-        out = self._new((T, H))
+        out = self._new((T, H)) if want_rows else None
         self._call("norm", "sl_add_postnorm", _p(resid), _p(y), _p(weight), _p(out), T, H, _c_float(eps),
                    _c_float(mult))
         return out
@@ -135,8 +135,35 @@ class RecurrentOps:
                    _c_float(unit_eps), scaled_heads, _c_float(scale), int(activation == "silu"), _p(out))
         return out
 
+    def stream_conv(self, resid, taps, state, state_off, batch, write, y=None, y_weight=None, y_eps=1e-6):
+        """Rows x_t + sum_j taps[j] x_(t - n + 1 + j) of the float32 stream x, per channel, in the
+        activation dtype (``taps`` [n, width], the last one the token's own).  The n - 1 stream rows
+        before a step come from the sequence's state slot at ``state_off`` ([n - 1, width], zeros at a
+        sequence's start), and the step's last n - 1 go back there when ``write``.  ``y``: a sublayer's
+        output that first joins the stream, x += y / sqrt(mean(y^2) + y_eps) * y_weight, in place: in
+        the same launch when every sequence of the step has one token."""
+        T, H = resid.shape
+        self._check(resid, torch.float32, None, "residual stream")
+        n = taps.shape[0]
+        self._check(taps, torch.float32, (n, H), "taps")
+        self._sequences(batch, T)
+        slot_size = self._state(state, state_off + (n - 1) * H)
+        single = batch.max_q_len == 1
+        if y is not None:
+            self._check(y, self.act_dtype, (T, H), "sublayer output")
+            self._check(y_weight, torch.float32, (H,), "output norm weight")
+            if not single:
+                self.add_postnorm(resid, y, y_weight, y_eps, 1.0, want_rows=False)
+                y = None
+        out = self._new((T, H))
+        self._call(self._lazy("recurrent"), "sl_stream_conv", _p(resid), H, n, _p(taps), _p(state), _ll(slot_size),
+                   state_off, _p(batch.cu_q), _p(batch.positions), _p(batch.tok_seq), _p(batch.state_slots),
+                   batch.num_seqs, T, int(bool(write)), int(single), _p(y), _p(y_weight) if y is not None else None,
+                   _c_float(y_eps), _p(out))
+        return out
+
     def _scan(self, mode, src, q_col, k_col, v_col, H, G, D, Dv, log_decay, q_scale, gates, i_col, f_col,
-              cap, state, batch, write, rates=None, step_bias=None, skip=None):
+              cap, state, batch, write, rates=None, step_bias=None, skip=None, lower=None):
         T, stride = self._f32_rows(src, "q, k, v rows")
         self._sequences(batch, T)
         need = H * Dv * D + (H * D + H if mode == _SCAN_LSTM else 0)
@@ -151,7 +178,8 @@ class RecurrentOps:
         out = self._new((T, H * Dv), torch.float32)
         self._call(self._lazy("recurrent"), "sl_matrix_scan", mode, _p(src), stride, q_col, k_col, v_col, H, G,
                    D, Dv, _p(log_decay), _c_float(q_scale), _p(gates), gate_stride, i_col, f_col, _c_float(cap),
-                   _p(rates), _p(step_bias), _p(skip), _p(state), _ll(slot_size), _p(batch.cu_q), _p(batch.positions), _p(batch.state_slots),
+                   _p(rates), _p(step_bias), _p(skip), _p(lower), _p(state), _ll(slot_size), _p(batch.cu_q),
+                   _p(batch.positions), _p(batch.state_slots),
                    batch.num_seqs, T, int(bool(write)), _p(out))
         return out
 
@@ -187,18 +215,28 @@ class RecurrentOps:
         return self._scan(_SCAN_SSD, src, c_col, b_col, x_col, H, G, N, P, None, 1.0, steps, step_col, 0, 1.0,
                           state, batch, write, rates=rates, step_bias=step_bias, skip=skip)
 
-    def head_norm_gate(self, o, H, Dv, weight, per_head, eps, gate, gate_col, activation, gate_first=False):
+    def forget_scan(self, buf, q_col, f_col, v_col, H, D, Dv, lower, state, batch, write, q_scale=1.0):
+        """Linear attention whose forget gate also writes: with f = lower + (1 - lower) sigmoid(z), z at
+        column ``f_col`` of ``buf`` (float32 rows, biases included) and ``lower`` [H D], per head
+        S' = diag(f) S + (1 - f) v^T and o = S'^T (q_scale silu(q)).  The slot holds S as [H, Dv, D] from
+        0 on; a sequence whose first token is in the step starts from zero.  Returns float32 [T, H Dv]."""
+        self._check(lower, torch.float32, (H * D,), "lower bounds")
+        return self._scan(_SCAN_FORGET, buf, q_col, f_col, v_col, H, H, D, Dv, None, q_scale, None, 0, 0, 1.0,
+                          state, batch, write, lower=lower)
+
+    def head_norm_gate(self, o, H, Dv, weight, per_head, eps, gate=None, gate_col=0, activation="sigmoid",
+                       gate_first=False):
         """Each head of ``o`` [T, H Dv] (float32) divided by its root mean square, times ``weight``
         ([H Dv] when ``per_head``, else [Dv] for every head), times sigmoid or silu of
         gate[:, gate_col + h Dv + d] (float32 rows).  ``gate_first``: the gate is applied before the
-        norm (a "head" is then any equal part of the row that is normed by itself).  Returns rows in
-        the activation dtype."""
+        norm (a "head" is then any equal part of the row that is normed by itself).  ``gate`` None: the
+        norm alone.  Returns rows in the activation dtype."""
         T, width = self._f32_rows(o, "read-out")
         if width != H * Dv:
             raise KernelError("head_norm_gate: the read-out is not [T, heads * channels]")
         self._check(weight, torch.float32, (H * Dv if per_head else Dv,), "gain")
-        gate_stride = self._f32_rows(gate, "gates")[1]
-        if gate.shape[0] != T or activation not in ("sigmoid", "silu"):
+        gate_stride = self._f32_rows(gate, "gates")[1] if gate is not None else 0
+        if (gate is not None and gate.shape[0] != T) or activation not in ("sigmoid", "silu"):
             raise KernelError("head_norm_gate: gates for another number of tokens, or an unknown activation")
         out = self._new((T, H * Dv))
         self._call(self._lazy("recurrent"), "sl_head_norm_gate", _p(o), T, H, Dv, _p(weight), int(bool(per_head)),
@@ -210,12 +248,13 @@ class RecurrentOps:
     CONV_IN_STORE_MAX_CHANNELS = 12288    # (a token's convolved row waits in 48 KB of LDS)
 
     def projnorm_rope_store(self, buf, H, G, D, Dv, q_gain, k_gain, eps, rot, tables, slots, k_cache, v_cache,
-                            page_size, values_are_keys=False, conv=None):
+                            page_size, values_are_keys=False, conv=None, per_head=False):
         """``buf`` (float32) holds q [H D], k [G D] and v [G Dv] side by side.  q and k are
         RMS-normed over all their heads at once (gains of that size; both None: no norm), the first ``rot`` channels of
         every head rotated in halves by ``tables``; k and v go to the token's place in the pages
         (``slots`` None: no write); q comes back as [T, H D] in the activation dtype.
-        ``values_are_keys``: there is no v in ``buf``; the values cached are the keys as they lie
+        ``per_head``: q and k are normed head by head instead (gains of the same sizes, so a gain may
+        differ from head to head).  ``values_are_keys``: there is no v in ``buf``; the values cached are the keys as they lie
         in ``buf``, before norm and rotation (Dv = D).  ``conv`` = (taps [C, n], state, state_off, batch,
         write): q, k and v (the row's first C channels) first pass the short causal convolution of
         ``short_conv`` without bias and activation, in the same launch; the state's last inputs are
@@ -244,7 +283,7 @@ class RecurrentOps:
             self._check(slots, torch.int32, (T,), "slots")
         q = self._new((T, H * D))
         self._call(self._lazy("recurrent"), "sl_projnorm_rope_store", _p(buf), stride, T, H, G, D, Dv, _p(q_gain),
-                   _p(k_gain), _c_float(eps), rot, _p(cos), _p(sin), _p(slots),
+                   _p(k_gain), _c_float(eps), int(bool(per_head)), rot, _p(cos), _p(sin), _p(slots),
                    _p(k_cache) if slots is not None else None, _p(v_cache) if slots is not None else None,
                    page_size, _p(q), H * D if values_are_keys else (H + G) * D, *self._conv_args(conv, T, stride))
         return q

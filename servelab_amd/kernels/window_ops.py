@@ -184,7 +184,7 @@ class WindowOps:
     # ------------------------------------------------------------ attention
     def window_attention(self, q, q_col, nh, nkv, Dk, Dv, k_cache, v_cache, page_size, block_tables,
                          batch, scale, window, keep_first=0, slopes=None, sinks=None, gate=None,
-                         gate_col=0, softcap=None):
+                         gate_col=0, softcap=None, channel_gate=None, channel_gate_col=0):
         """Attention of every token of the batch over its sequence's pages.  ``q`` [T, width]
         holds head h of a token at column ``q_col + h * Dk``; ``v_cache`` None: values are the
         first Dv channels of the key rows.  ``window`` (None: all keys) and ``keep_first``: the
@@ -192,7 +192,8 @@ class WindowOps:
         [nh]: slope_h * (i - j) is taken off the scaled score; ``sinks`` [nh]: exp(sink_h) joins
         the denominator; ``gate`` [T, width] with head h's gate at column ``gate_col + h``: the
         output is multiplied by its sigmoid.  ``softcap`` c: the scaled score s becomes
-        c tanh(s / c).  Returns [T, nh * Dv]."""
+        c tanh(s / c).  ``channel_gate`` (float32 rows [T, width]): the output's channel d of head h is
+        multiplied by the sigmoid of column ``channel_gate_col + h * Dv + d``.  Returns [T, nh * Dv]."""
         T = q.shape[0]
         S, max_pages = block_tables.shape
         self._check(q, self.act_dtype, None, "q")
@@ -220,6 +221,12 @@ class WindowOps:
             if gate.dim() != 2 or gate.shape[0] != T or gate_col < 0 or gate_col + nh > gate.shape[1]:
                 raise KernelError("window_attention: the gates do not fit their rows")
             gate_stride = gate.shape[1]
+        channel_stride = 0
+        if channel_gate is not None:
+            self._check(channel_gate, torch.float32, None, "channel gate")
+            channel_stride = channel_gate.shape[1] if channel_gate.dim() == 2 else 0
+            if channel_gate.shape[0] != T or channel_gate_col < 0 or channel_gate_col + nh * Dv > channel_stride:
+                raise KernelError("window_attention: the channel gates do not fit their rows")
         window = int(window or 0)
         # shares of the keys: for steps of single tokens only, by the number of keys a token can see
         # there; fixed by sizes that a captured step keeps.  (A prompt's tiles are not cut: measured at
@@ -255,5 +262,6 @@ class WindowOps:
                    _c_float(float(softcap or 0.0)), window,
                    int(keep_first), _p(slopes), _p(sinks),
                    _c_void_p(gate.data_ptr() + gate_col * item) if gate is not None else None, gate_stride,
-                   _p(out), nsplit, _p(part_o), _p(part_ml))
+                   _c_void_p(channel_gate.data_ptr() + 4 * channel_gate_col) if channel_gate is not None else None,
+                   channel_stride, _p(out), nsplit, _p(part_o), _p(part_ml))
         return out

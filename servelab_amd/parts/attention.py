@@ -119,19 +119,31 @@ class ProjectionNormAttention(Mixer):
     in the checkpoint); ``bias`` False: no biases.  ``values`` "keys": there is no value
     projection; a token's values are its keys as the projection left them (with their bias),
     before norm and rotation.  ``softcap`` c: a scaled score s becomes c tanh(s / c).
+    ``projection_norm`` "head": every head of q and k is normed by itself, with one gain of
+    ``key_dim`` channels for all heads.  ``temperature``: head h's scores are multiplied by a stored
+    number of its own (it joins the gain of q, in float32).  ``gate`` "channel": the heads' outputs are
+    multiplied, channel by channel, by the sigmoid of a further projection of the input.
+    ``out_bias`` (None: as ``bias``): whether the output projection has one.
     The input goes to nothing but the input product and the output product's result only joins the
     stream, so in steps of few rows a pre-norm block's norms can run the products around them."""
     graph_safe = True
     takes_scaled_rows = True
 
     NAMES = {"q": "q", "k": "k", "v": "v", "out": "o", "q_bias": "q.b", "k_bias": "k.b",
-             "v_bias": "v.b", "out_bias": "o.b", "q_norm": "q.norm", "k_norm": "k.norm"}
+             "v_bias": "v.b", "out_bias": "o.b", "q_norm": "q.norm", "k_norm": "k.norm",
+             "temperature": "temp", "gate": "g"}
 
     def __init__(self, hidden_size, num_heads, num_kv_heads, key_dim, value_dim, scale, position,
                  norm_eps, bias=True, window=None, names=None, projection_norm=True, values="projected",
-                 softcap=None):
+                 softcap=None, temperature=False, gate=None, out_bias=None):
         if num_heads % num_kv_heads:
             raise ValueError("num_heads must be a multiple of num_kv_heads")
+        if projection_norm not in (True, False, "head"):
+            raise ValueError("projection_norm is True (over all heads), 'head' or False")
+        if gate not in (None, "channel"):
+            raise ValueError("the gate is None or 'channel'")
+        if temperature and not projection_norm:
+            raise ValueError("the factor per head is kept in the gain of q's norm")
         if values not in ("projected", "keys"):
             raise ValueError("values are 'projected' or 'keys'")
         self.hidden_size = int(hidden_size)
@@ -143,14 +155,17 @@ class ProjectionNormAttention(Mixer):
         self.scale, self.norm_eps = float(scale), float(norm_eps)
         self.position = position
         self.bias = bool(bias)
+        self.out_bias = self.bias if out_bias is None else bool(out_bias)
         self.projection_norm = bool(projection_norm)
+        self.head_norm = projection_norm == "head"
+        self.temperature, self.gate = bool(temperature), gate
         self.window = None if not window else int(window)
         self.softcap = float(softcap) if softcap else None
         self.names = dict(self.NAMES, **(names or {}))
 
     @property
     def in_channels(self):
-        """Channels of the input projection: q, k and (with a value projection) v."""
+        """Channels of the input projection before the gate's: q, k and (with a value projection) v."""
         H, G, D, Dv = self.num_heads, self.num_kv_heads, self.key_dim, self.value_dim
         return (H + G) * D + (0 if self.values_are_keys else G * Dv)
 
@@ -161,13 +176,18 @@ class ProjectionNormAttention(Mixer):
         if not self.values_are_keys:
             specs[n["v"]] = ParamSpec((G * Dv, h))
         if self.projection_norm:
-            specs.update({n["q_norm"]: ParamSpec((H * D,), init="gain"),
-                          n["k_norm"]: ParamSpec((G * D,), init="gain")})
+            specs.update({n["q_norm"]: ParamSpec((D if self.head_norm else H * D,), init="gain"),
+                          n["k_norm"]: ParamSpec((D if self.head_norm else G * D,), init="gain")})
         if self.bias:
-            specs.update({n["q_bias"]: ParamSpec((H * D,)), n["k_bias"]: ParamSpec((G * D,)),
-                          n["out_bias"]: ParamSpec((h,))})
+            specs.update({n["q_bias"]: ParamSpec((H * D,)), n["k_bias"]: ParamSpec((G * D,))})
             if not self.values_are_keys:
                 specs[n["v_bias"]] = ParamSpec((G * Dv,))
+        if self.out_bias:
+            specs[n["out_bias"]] = ParamSpec((h,))
+        if self.temperature:
+            specs[n["temperature"]] = ParamSpec((H,), init="gain")
+        if self.gate:
+            specs[n["gate"]] = ParamSpec((H * Dv, h))
         return specs
 
     def cache_spec(self):
@@ -191,6 +211,8 @@ class ProjectionNormAttention(Mixer):
         rows = [self._by_head(tensors(n["q"]), H), self._by_head(tensors(n["k"]), G)]
         if not self.values_are_keys:
             rows.append(tensors(n["v"]))
+        if self.gate:
+            rows.append(tensors(n["gate"]))
         w = torch.cat(rows, 0)
         extra = -w.shape[0] % 8
         if extra:
@@ -201,14 +223,25 @@ class ProjectionNormAttention(Mixer):
             b = [self._by_head(tensors(n["q_bias"]).float(), H), self._by_head(tensors(n["k_bias"]).float(), G)]
             if not self.values_are_keys:
                 b.append(tensors(n["v_bias"]).float())
-            self.b_in = rt.vector(torch.cat(b + [torch.zeros(extra, device=w.device)], 0))
+            b.append(torch.zeros(w.shape[0] - self.in_channels, device=w.device))
+            self.b_in = rt.vector(torch.cat(b, 0))
+        if self.out_bias:
             self.b_o = rt.vector(tensors(n["out_bias"]))
-        self.q_gain = rt.vector(self._by_head(tensors(n["q_norm"]), H)) if self.projection_norm else None
-        self.k_gain = rt.vector(self._by_head(tensors(n["k_norm"]), G)) if self.projection_norm else None
+        self.q_gain = self.k_gain = None
+        if self.projection_norm:
+            q_gain, k_gain = tensors(n["q_norm"]).float(), tensors(n["k_norm"]).float()
+            if self.head_norm:
+                q_gain, k_gain = q_gain.repeat(H), k_gain.repeat(G)
+            if self.temperature:
+                q_gain = q_gain * tensors(n["temperature"]).float().repeat_interleave(D)
+            self.q_gain = rt.vector(self._by_head(q_gain, H))
+            self.k_gain = rt.vector(self._by_head(k_gain, G))
         w_o = tensors(n["out"])
         if self.values_are_keys:
             # the values arrive in the keys' order: the output projection's columns follow them
             w_o = w_o.reshape(w_o.shape[0], H, Dv)[:, :, self.order.to(w_o.device)].reshape(w_o.shape)
+            if self.gate and layout is not None and layout.pairing != "half":
+                raise ValueError("a channel gate over keys that turn in neighbouring pairs is not supported")
         self.w_o = rt.linear_weight(w_o, delta=True)
 
     def forward(self, x, batch, cache, shared):
@@ -229,10 +262,17 @@ class ProjectionNormAttention(Mixer):
             more["values_are_keys"] = True
         if conv is not None:
             more["conv"] = conv
+        if self.head_norm:
+            more["per_head"] = True
         q = ops.projnorm_rope_store(*store, **more)
         attend = (q, 0, H, G, D, Dv, cache.k, cache.v, cache.page_size, group.block_tables, batch, self.scale,
                   self.window)
-        attn = ops.window_attention(*attend, softcap=self.softcap) if self.softcap else ops.window_attention(*attend)
+        options = {}
+        if self.softcap:
+            options["softcap"] = self.softcap
+        if self.gate:
+            options.update(channel_gate=buf, channel_gate_col=self.in_channels)
+        attn = ops.window_attention(*attend, **options)
         return ops.linear(attn, self.w_o, self.b_o, defer=True)
 
 

@@ -18,6 +18,7 @@ embedding output side by side, plus a vector of the pass: what a stretch of laye
 several times starts every pass with.
 """
 from .base import Block, prefixed
+from .norm import NormedDelta
 
 
 class PreNormBlock(Block):
@@ -157,11 +158,18 @@ class PostNormBlock(Block):
     declares its cache needs as a list (``cache_specs``) and gets the list of bindings.
 
     The rows of the stream travel from block to block in the step's ``shared`` dict; a block of
-    another kind that changes the stream has to drop the entry ``"stream rows"``."""
+    another kind that changes the stream has to drop the entry ``"stream rows"``.
 
-    def __init__(self, norm1, mixer, norm2, feedforward, names=("norm1.", "mix.", "norm2.", "mlp.")):
+    ``input_conv`` (a ``StreamConvolution``): the mixer reads the stream plus a convolution over time of
+    it, Mixer(h + Conv(h)).  Such a block keeps the convolution's last inputs (its first cache need)
+    and leaves its last output with the norm it has to pass (``NormedDelta``), which the next block's
+    convolution, or the final norm, adds to the stream in its own kernel call."""
+
+    def __init__(self, norm1, mixer, norm2, feedforward, names=("norm1.", "mix.", "norm2.", "mlp."),
+                 input_conv=None, conv_name=""):
         self.norm1, self.mixer, self.norm2, self.feedforward = norm1, mixer, norm2, feedforward
         self.names = tuple(names)
+        self.input_conv, self.conv_name = input_conv, conv_name
 
     @property
     def graph_safe(self):
@@ -171,14 +179,17 @@ class PostNormBlock(Block):
         parts = [(self.names[0], self.norm1), (self.names[1], self.mixer)]
         if self.feedforward is not None:
             parts += [(self.names[2], self.norm2), (self.names[3], self.feedforward)]
+        if self.input_conv is not None:
+            parts.append((self.conv_name, self.input_conv))
         return parts
 
     def cache_specs(self):
+        specs = self.input_conv.cache_specs() if self.input_conv is not None else []
         several = getattr(self.mixer, "cache_specs", None)
         if several is not None:
-            return list(several())
+            return specs + list(several())
         spec = self.mixer.cache_spec()
-        return [] if spec is None else [spec]
+        return specs if spec is None else specs + [spec]
 
     def param_specs(self):
         specs = {}
@@ -195,17 +206,30 @@ class PostNormBlock(Block):
     def forward(self, resid, delta, batch, caches, shared):
         ops = self.rt.ops
         x = shared.get("stream rows")
-        if delta is not None:                 # what a block of another kind left to be added
+        if delta is not None and not (isinstance(delta, NormedDelta) and self.input_conv is not None):
+            # what a block of another kind left to be added
             for d in (delta if isinstance(delta, (tuple, list)) else (delta,)):
-                if d is not None:
+                if isinstance(d, NormedDelta):
+                    ops.add_postnorm(resid, d.y, d.weight, d.eps, 1.0, want_rows=False)
+                elif d is not None:
                     ops.add_into(resid, ops.materialize(d))
-            x = None
-        if x is None:
+            x = delta = None
+        if self.input_conv is not None:
+            kept = len(self.input_conv.cache_specs())
+            x = self.input_conv.forward(resid, delta, batch, caches[0] if kept else None)
+            caches = caches[kept:]
+            shared.pop("stream rows", None)
+        elif x is None:
             x = self.norm1.forward_post(resid, None)
         if hasattr(self.mixer, "cache_specs"):
             y = self.mixer.forward(x, batch, caches, shared)
         else:
             y = self.mixer.forward(x, batch, caches[0] if caches else None, shared)
+        if self.input_conv is not None:
+            if self.feedforward is None:
+                return self.norm1.normed(y)
+            x = self.norm1.forward_post(resid, ops.materialize(y))
+            return self.norm2.normed(self.feedforward.forward(x))
         x = self.norm1.forward_post(resid, ops.materialize(y))
         if self.feedforward is not None:
             x = self.norm2.forward_post(resid, ops.materialize(self.feedforward.forward(x)))

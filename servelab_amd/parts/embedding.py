@@ -10,22 +10,32 @@ from .base import Embedding, Part, ParamSpec
 class TokenEmbedding(Embedding):
     graph_safe = True
 
-    def __init__(self, vocab_size: int, hidden_size: int, name: str = "weight", scale: float = 1.0):
-        """``scale``: the rows of the table enter the stream multiplied by it (in float32)."""
+    def __init__(self, vocab_size: int, hidden_size: int, name: str = "weight", scale: float = 1.0,
+                 positions: int = 0, position_name: str = "positions"):
+        """``scale``: the rows of the table enter the stream multiplied by it (in float32).
+        ``positions`` P: a learned vector of the token's position, out of a table [P, H], is added
+        (unscaled); no sequence may then be longer than P."""
         self.vocab_size, self.hidden_size = int(vocab_size), int(hidden_size)
         self.name = name
         self.scale = float(scale)
+        self.positions, self.position_name = int(positions), position_name
 
     def param_specs(self):
-        return {self.name: ParamSpec((self.vocab_size, self.hidden_size))}
+        specs = {self.name: ParamSpec((self.vocab_size, self.hidden_size))}
+        if self.positions:
+            specs[self.position_name] = ParamSpec((self.positions, self.hidden_size))
+        return specs
 
     def load(self, tensors, rt):
         self.rt = rt
         self.weight = rt.matrix(tensors(self.name))
+        self.position_table = rt.matrix(tensors(self.position_name)) if self.positions else None
 
     def forward(self, batch):
         """The rows of the table at ``batch.ids`` (int32 [T]) as the float32
         residual stream [T, H]."""
+        if self.position_table is not None:
+            return self.rt.ops.embed(batch.ids, self.weight, self.scale, batch.positions, self.position_table)
         if self.scale != 1.0:
             return self.rt.ops.embed(batch.ids, self.weight, self.scale)
         return self.rt.ops.embed(batch.ids, self.weight)

@@ -89,4 +89,4 @@ class PlainMLP(FeedForward):
 
     def forward(self, x):
         ops = self.rt.ops
-        return ops.linear(ops.activate(ops.linear(x, self.w_up, None), self.activation), self.w_down, None)
+        return ops.plain_mlp(x, self.w_up, self.w_down, self.activation, defer=True)

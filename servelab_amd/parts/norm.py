@@ -91,5 +91,12 @@ class PostRMSNorm(RMSNorm):
         super().__init__(size, eps, name)
         self.mult = float(mult)
 
+    def load(self, tensors, rt):
+        super().load(tensors, rt)
+        self.delta_weight = self.weight if self.mult == 1.0 else (self.weight * self.mult).contiguous()
+
+    def normed(self, y):
+        return NormedDelta(self.rt.ops.materialize(y), self.delta_weight, self.eps)
+
     def forward_post(self, resid, y):
         return self.rt.ops.add_postnorm(resid, y, self.weight, self.eps, self.mult)

@@ -25,6 +25,10 @@ and silu; dt = softplus(dt~ + dt_bias_h); S' = exp(-exp(A_log_h) dt) S + dt B x^
 the whole head), y = S'^T C + D_h x; y times silu(z), then RMS-normed in equal parts with a gain
 over the whole row.  The convolution's last taps - 1 inputs are part of the state.
 
+``BoundedForgetAttention`` (HGRN2): a forget gate per key channel that also says how much is written,
+f = l + (1 - l) sigmoid(z) with a stored lower bound l: S' = diag(f) S + (1 - f) v^T, read by silu(q);
+o RMS-normed per head with a gain shared by the heads, no output gate.
+
 Gates, decays, unit norms, state and read-out are float32 in both activation types; the input
 projection (one product for everything a mixer projects from its input) returns float32 sums.
 A state starts from zero at a sequence's first token, whatever the slot held.  Every size and
@@ -270,6 +274,39 @@ class StateSpaceMixer(_MatrixMemoryMixer):
         y = ops.head_norm_gate(y, self.norm_groups, self.inner // self.norm_groups, self.gain, True,
                                self.norm_eps, buf, at["z"], "silu", gate_first=True)
         return ops.linear(y, self.w_o, None)
+
+
+class BoundedForgetAttention(_MatrixMemoryMixer):
+    NAMES = {"q": "q", "f": "f", "f_bias": "f.b", "lower": "lower", "v": "v", "norm": "norm", "out": "o"}
+
+    def __init__(self, hidden_size, heads, dim, vdim, norm_eps, names=None):
+        self.hidden_size, self.heads, self.dim, self.vdim = int(hidden_size), int(heads), int(dim), int(vdim)
+        self.norm_eps = float(norm_eps)
+        self.names = dict(self.NAMES, **(names or {}))
+
+    def param_specs(self):
+        n, h, H, D, Dv = self.names, self.hidden_size, self.heads, self.dim, self.vdim
+        return {n["q"]: ParamSpec((H * D, h)), n["f"]: ParamSpec((H * D, h)), n["f_bias"]: ParamSpec((H * D,)),
+                n["lower"]: ParamSpec((H * D,), init="normal"), n["v"]: ParamSpec((H * Dv, h)),
+                n["norm"]: ParamSpec((Dv,), init="gain"), n["out"]: ParamSpec((h, H * Dv))}
+
+    def cache_spec(self):
+        return StateSpec((self.heads * self.dim * self.vdim,), "float32")
+
+    def load(self, tensors, rt):
+        self.rt = rt
+        n = self.names
+        self._load_in([(x, tensors(n[x])) for x in ("q", "f", "v")], rt, {"f": tensors(n["f_bias"])})
+        self.lower = rt.vector(tensors(n["lower"]))
+        self.gain = rt.vector(tensors(n["norm"]))
+        self.w_o = rt.linear_weight(tensors(n["out"]), delta=True)
+
+    def forward(self, x, batch, cache, shared):
+        ops, at = self.rt.ops, self.at
+        H, D, Dv = self.heads, self.dim, self.vdim
+        buf = self._project(x)
+        o = ops.forget_scan(buf, at["q"], at["f"], at["v"], H, D, Dv, self.lower, cache.state, batch, cache.write)
+        return ops.linear(ops.head_norm_gate(o, H, Dv, self.gain, False, self.norm_eps), self.w_o, None)
 
 
 class SideBySide(Mixer):

@@ -22,8 +22,9 @@ class EmulatedOps:
         self.act_dtype = act_dtype
 
     # ------------------------------------------------------------ embedding
-    def embed(self, ids, table, scale=1.0):
-        return _f(table[ids.long()]) * scale
+    def embed(self, ids, table, scale=1.0, positions=None, pos_table=None):
+        out = _f(table[ids.long()]) * scale
+        return out if pos_table is None else out + _f(pos_table[positions.long()])
 
     def stream_pair(self, resid, delta, other):
         """[resid + delta | other] as rows in the activation dtype; the streams stay as they are."""
@@ -97,6 +98,16 @@ class EmulatedOps:
                   bias_down=None):
         return self.linear(self.gated_linear(x, w_gate_up, block, activation, bias_gate_up), w_down, bias_down,
                            defer=defer)
+
+    def activated_linear(self, x, w, activation, bias=None):
+        """(bfloat16 on the device: few rows are activated before the rounding, many after it)"""
+        y = _f(x) @ _f(w).T
+        if bias is not None:
+            y = y + bias
+        return self._act(y, activation).to(self.act_dtype)
+
+    def plain_mlp(self, x, w_up, w_down, activation, defer=False):
+        return self.linear(self.activated_linear(x, w_up, activation), w_down, None, defer=defer)
 
     def gated_linear(self, x, w, block, activation="silu", bias=None):
         """(the kernels apply the gate to float32 sums; so does this)"""
@@ -210,13 +221,20 @@ class EmulatedOps:
     def add_into(self, resid, delta):
         resid += _f(delta)
 
-    def add_postnorm(self, resid, y, weight, eps, mult):
+    def add_postnorm(self, resid, y, weight, eps, mult, want_rows=True):
         """resid += mult * y / sqrt(mean(y^2) + eps) * weight; returns the stream's rows in the
-        activation dtype (y None: only those)."""
+        activation dtype (y None: only those; want_rows False: None)."""
         if y is not None:
             y = _f(y)
             resid += mult * (y * torch.rsqrt(y.pow(2).mean(-1, keepdim=True) + eps) * weight)
-        return resid.to(self.act_dtype)
+        return resid.to(self.act_dtype) if want_rows else None
+
+    def stream_conv(self, resid, taps, state, state_off, batch, write, y=None, y_weight=None, y_eps=1e-6):
+        """resid += the normed y (if given); then rows x_t + sum_j taps[j] x_(t - n + 1 + j) of the stream x
+        (taps [n, width]); the n - 1 rows before a step lie in state[slot, state_off:] as [n - 1, width]."""
+        if y is not None:
+            self.add_postnorm(resid, y, y_weight, y_eps, 1.0, want_rows=False)
+        return (resid + self.short_conv(resid, 0, taps.T, state, state_off, batch, write, activation=None)).to(self.act_dtype)
 
     def scaled_sum(self, a, sa, b, sb):
         return (sa * _f(a) + sb * _f(b)).to(self.act_dtype)
@@ -357,12 +375,36 @@ class EmulatedOps:
                 kept.copy_(S)
         return out.view(T, H * P)
 
-    def head_norm_gate(self, o, H, Dv, weight, per_head, eps, gate, gate_col, activation, gate_first=False):
+    def forget_scan(self, buf, q_col, f_col, v_col, H, D, Dv, lower, state, batch, write, q_scale=1.0):
+        """f = lower + (1 - lower) sigmoid(z), z at column f_col; S' = diag(f) S + (1 - f) v^T and o = S'^T
+        (q_scale silu(q)).  The slot holds S as [H, Dv, D] from 0 on."""
+        T = buf.shape[0]
+        q = buf[:, q_col:q_col + H * D].float().view(T, H, D)
+        q = q * torch.sigmoid(q) * q_scale
+        z = buf[:, f_col:f_col + H * D].float().view(T, H, D)
+        l = lower.view(H, D)
+        keep, add = l + (1 - l) * torch.sigmoid(z), (1 - l) * torch.sigmoid(-z)
+        v = buf[:, v_col:v_col + H * Dv].float().view(T, H, Dv)
+        out = torch.empty(T, H, Dv)
+        for a, b, slot, fresh in self._sequences(batch):
+            kept = state[slot, :H * Dv * D].view(H, Dv, D)
+            S = torch.zeros(H, Dv, D) if fresh else kept.clone()
+            for t in range(a, b):
+                S = S * keep[t][:, None, :] + v[t][:, :, None] * add[t][:, None, :]
+                out[t] = torch.einsum("hvd,hd->hv", S, q[t])
+            if write:
+                kept.copy_(S)
+        return out.view(T, H * Dv)
+
+    def head_norm_gate(self, o, H, Dv, weight, per_head, eps, gate=None, gate_col=0, activation="sigmoid",
+                       gate_first=False):
         """Each head of o [T, H Dv] (float32) divided by its root mean square, times ``weight``
         ([H Dv] when ``per_head``, else [Dv] for every head), times sigmoid or silu of
         gate[:, gate_col:gate_col + H Dv]."""
         T = o.shape[0]
         x = o.view(T, H, Dv)
+        if gate is None:            # the norm alone
+            gate, gate_col = torch.full((T, H * Dv), 40.0), 0
         g = gate[:, gate_col:gate_col + H * Dv].float().view(T, H, Dv)
         g = torch.sigmoid(g) if activation == "sigmoid" else g * torch.sigmoid(g)
         if gate_first:              # the gate before the norm
@@ -375,7 +417,7 @@ class EmulatedOps:
 
     # -------------------------------------- attention with a norm over the projection
     def projnorm_rope_store(self, buf, H, G, D, Dv, q_gain, k_gain, eps, rot, tables, slots, k_cache,
-                            v_cache, page_size, values_are_keys=False, conv=None):
+                            v_cache, page_size, values_are_keys=False, conv=None, per_head=False):
         """buf (float32) holds q [H D], k [G D], v [G Dv] side by side.  q and k are RMS-normed over
         all their heads at once, their heads' first ``rot`` channels rotated in halves; k and v go
         to the pages, q is returned [T, H D]."""
@@ -387,6 +429,9 @@ class EmulatedOps:
         def normed(x, gain):
             if gain is None:        # no norm over the projection
                 return x
+            if per_head:            # every head by itself
+                heads = x.view(T, -1, D)
+                return (heads * torch.rsqrt(heads.pow(2).mean(-1, keepdim=True) + eps)).view(T, -1) * gain
             return x * torch.rsqrt(x.pow(2).mean(-1, keepdim=True) + eps) * gain
 
         def turned(x):
@@ -408,7 +453,7 @@ class EmulatedOps:
 
     def window_attention(self, q, q_col, nh, nkv, Dk, Dv, k_cache, v_cache, page_size, block_tables,
                          batch, scale, window, keep_first=0, slopes=None, sinks=None, gate=None,
-                         gate_col=0, softcap=None):
+                         gate_col=0, softcap=None, channel_gate=None, channel_gate_col=0):
         if slopes is not None or sinks is not None or gate is not None:
             raise NotImplementedError("the emulated window attention has no bias, sink or gate")
         T = q.shape[0]
@@ -437,6 +482,8 @@ class EmulatedOps:
                 scores = softcap * torch.tanh(scores / softcap)
             scores = scores.masked_fill(~vis[None], float("-inf"))
             o = torch.einsum("hqr,rhd->qhd", torch.softmax(scores, -1), v)
+            if channel_gate is not None:
+                o = o * torch.sigmoid(channel_gate[a:b, channel_gate_col:channel_gate_col + nh * Dv].view(b - a, nh, Dv))
             out[a:b] = o.reshape(b - a, nh * Dv).to(self.act_dtype)
         return out
 
