@@ -194,10 +194,36 @@ def vunadra_configs(shape, layers, window):
     return vunadra, futezen_configs(shape, layers)[0]
 
 
+def kelutar_configs(shape, layers, window, positions):
+    """(Kelutar config.json, Vekanex config.json) of equal size: Vekanex is the design nearest to it (norms
+    on the sublayers' outputs, a matrix per head in a state slot, layers that run again).  Kelutar's layers
+    come in the order linear attention with a bounded forget gate, softmax attention over a window, linear
+    attention, and the first layer's weights once more, each behind a convolution of 4 taps; memory heads
+    as Vekanex's, the attention's heads as the shape's, dense feed-forwards of the shape's width."""
+    z, v = DESIGN_SHAPES[shape], VEKANEX_SHAPES[shape]
+    mlp = {"kind": "dense", "ff": z["ff"]}
+    memory = {"type": "hgrn2", "mlp": mlp,
+              "mixer": {"heads": v["memory_heads"], "dim": v["memory_dim"], "vdim": v["memory_vdim"]}}
+    att = {"type": "attention", "mlp": mlp,
+           "mixer": {"heads": z["heads"], "kv_heads": z["kv_heads"], "dim": z["dim"], "vdim": z["dim"],
+                     "scale": z["dim"] ** -0.5, "mask": {"size": window}}}
+    order = [memory, att, memory, dict(memory, weights_of=0)]
+    listed = []
+    for i in range(layers):
+        entry = order[i % 4]
+        if "weights_of" in entry:
+            entry = dict(entry, weights_of=i - 3)
+        listed.append(entry)
+    kelutar = {"architecture": "Kelutar", "width": z["width"], "vocab": z["vocab"], "max_positions": positions,
+               "norm": {"eps": 1e-5}, "embedding": {"scale": z["width"] ** 0.5}, "canon": {"taps": 4},
+               "torch_dtype": "bfloat16", "layers": listed}
+    return kelutar, vekanex_configs(shape, layers)[0]
+
+
 def compare_designs(args):
     """Prefill and decode throughput of the design named by --design beside the Qwen2 decoder of equal
-    size (Futezen: beside the Vekanex decoder of equal size; Vunadra: beside the Futezen one), at each of --design-shapes: one JSON line,
-    tokens per second each."""
+    size (Futezen and Kelutar: beside the Vekanex decoder of equal size; Vunadra: beside the Futezen one),
+    at each of --design-shapes: one JSON line, tokens per second each."""
     import torch
     import servelab_amd  # noqa: F401
     from servelab_amd.config import resolve_architecture
@@ -210,8 +236,10 @@ def compare_designs(args):
                       "prefill_chunk": args.prefill_chunk, "page_size": page}, "shapes": {}}
     for shape in args.design_shapes.split(","):
         row = {}
-        other = "vekanex" if args.design == "futezen" else "futezen" if args.design == "vunadra" else "qwen2"
-        pair = vunadra_configs(shape, args.design_layers, args.design_window) if args.design == "vunadra" else \
+        other = {"futezen": "vekanex", "kelutar": "vekanex", "vunadra": "futezen"}.get(args.design, "qwen2")
+        pair = kelutar_configs(shape, args.design_layers, args.design_window,
+                               2 * max(args.context, args.prefill_tokens)) if args.design == "kelutar" else \
+            vunadra_configs(shape, args.design_layers, args.design_window) if args.design == "vunadra" else \
             futezen_configs(shape, args.design_layers) if args.design == "futezen" else \
             vekanex_configs(shape, args.design_layers) if args.design == "vekanex" else \
             design_configs(shape, args.design_layers, args.design_window)
@@ -380,7 +408,7 @@ def main():
     ap.add_argument("--no-prefill", action="store_true")
     ap.add_argument("--no-tune", action="store_true",
                     help="leave the library's default kernel choice for the prompt products")
-    ap.add_argument("--design", default="", choices=["", "topelorn", "vekanex", "futezen", "vunadra"],
+    ap.add_argument("--design", default="", choices=["", "topelorn", "vekanex", "futezen", "vunadra", "kelutar"],
                     help="instead of the default workload: prefill and decode throughput of this design "
                          "beside the Qwen2 decoder of equal size")
     ap.add_argument("--design-shapes", default="3b,7b", help="comma-separated: " + ", ".join(sorted(DESIGN_SHAPES)))

@@ -158,10 +158,40 @@ __global__ void activate_kernel(const act_t* __restrict__ x, act_t* __restrict__
     out[i] = from_f<act_t>(sl_act(to_f(x[i]), act));
 }
 
+// The same in pieces of 16 bytes, two a thread (the whole buffer is a multiple of them and aligned).
+constexpr int ACT_PIECE = 16 / sizeof(act_t);
+struct __attribute__((aligned(16))) act_piece { act_t v[ACT_PIECE]; };
+template <int ACT>
+__global__ __launch_bounds__(256) void activate_pieces_kernel(const act_piece* x, act_piece* out, size_t n) {
+  const size_t i0 = (size_t)blockIdx.x * 512 + threadIdx.x;
+  act_piece p[2];
+#pragma unroll
+  for (int u = 0; u < 2; ++u)
+    if (i0 + u * 256 < n) p[u] = x[i0 + u * 256];
+#pragma unroll
+  for (int u = 0; u < 2; ++u) {
+    if (i0 + u * 256 >= n) continue;
+#pragma unroll
+    for (int j = 0; j < ACT_PIECE; ++j) p[u].v[j] = from_f<act_t>(sl_act(to_f(p[u].v[j]), ACT));
+    out[i0 + u * 256] = p[u];
+  }
+}
+
 extern "C" const char* sl_activate(const void* x, void* out, long long n, int act, hipStream_t stream) {
   SL_CHECK(n >= 0, "activate: the count must not be negative");
   SL_CHECK(act >= SL_ACT_SILU && act <= SL_ACT_GELU_TANH, "activate: unknown activation");
   if (n == 0) return nullptr;
+  const size_t pieces = (size_t)n / ACT_PIECE;
+  if (n % ACT_PIECE == 0 && (uintptr_t)x % 16 == 0 && (uintptr_t)out % 16 == 0 && (pieces + 511) / 512 <= 0x7fffffff) {
+    const unsigned grid = (unsigned)((pieces + 511) / 512);
+    const act_piece* src = (const act_piece*)x;
+    act_piece* dst = (act_piece*)out;
+    if (act == SL_ACT_SILU) activate_pieces_kernel<SL_ACT_SILU><<<grid, 256, 0, stream>>>(src, dst, pieces);
+    else if (act == SL_ACT_RELU) activate_pieces_kernel<SL_ACT_RELU><<<grid, 256, 0, stream>>>(src, dst, pieces);
+    else if (act == SL_ACT_RELU2) activate_pieces_kernel<SL_ACT_RELU2><<<grid, 256, 0, stream>>>(src, dst, pieces);
+    else activate_pieces_kernel<SL_ACT_GELU_TANH><<<grid, 256, 0, stream>>>(src, dst, pieces);
+    return sl_launch_status();
+  }
   const size_t blocks = ((size_t)n + 255) / 256;
   activate_kernel<<<(unsigned)(blocks < 262144 ? blocks : 262144), 256, 0, stream>>>((const act_t*)x, (act_t*)out,
                                                                                      (size_t)n, act);
