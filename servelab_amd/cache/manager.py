@@ -5,8 +5,9 @@ Reference: ``BlockManager`` without prefix cache
 (servelab/kv_cache/manager.py:153-227,306-316): one table per request serves
 all layers.  Here the cache streams of a model are grouped by what they need:
 streams that keep every key share one group, streams that keep a window of W
-keys share another, and each group has pages and block tables of its own.  A
-window group gives a page back as soon as no later query can see any of its
+keys share another, those that keep a chunk of C positions a third, and each group has
+pages and block tables of its own.  A
+window or chunk group gives a page back as soon as no later query can see any of its
 tokens.  Streams that need a fixed-size state per request get a slot, taken
 when the request opens and given back when it closes; the slot array exists
 even when no stream asks for state.
@@ -136,17 +137,18 @@ class CacheManager:
         return True
 
     def commit(self, request, total_tokens: int) -> None:
-        """Tokens [0, total_tokens) are now cached.  Window groups give back
+        """Tokens [0, total_tokens) are now cached.  Window and chunk groups give back
         the pages that no later query can see: a query at p >= total sees keys
-        r > p - W, so a page whose last token is <= total - W is dead, unless it
+        r > p - W (or from the start of the chunk p lies in), so a page whose tokens all
+        lie before that is dead, unless it
         holds one of the first ``keep_first`` tokens, which every query sees."""
         self.lengths[request] = total_tokens
         bs = self.page_size
         for g in self.page_groups:
-            if g.window is None:
+            if g.window is None and g.spec.chunk is None:
                 continue
             table = g.tables[request]
-            dead_pages = max(0, (total_tokens - g.window + 1) // bs)
+            dead_pages = g.spec.first_needed(total_tokens) // bs
             kept_pages = -(-g.spec.keep_first // bs)
             for j in range(kept_pages, min(dead_pages, len(table))):
                 if table[j] != RELEASED:

@@ -5,6 +5,7 @@ from .vekanex import VekanexConfig, VekanexLayer
 from .futezen import FutezenConfig, FutezenLayer
 from .vunadra import VunadraConfig, VunadraLayer
 from .kelutar import KelutarConfig, KelutarLayer
+from .lotinex import LotinexConfig, LotinexLayer
 from .engine import CacheConfig, SchedulerConfig, EngineConfig, PAGE_SIZES
 from .registry import (Architecture, register_architecture, registered_architectures,
                        resolve_architecture)

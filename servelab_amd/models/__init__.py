@@ -1,2 +1,2 @@
 """Importing this package registers the architectures it holds."""
-from . import futezen, kelutar, qwen2, topelorn, vekanex, vunadra  # noqa: F401
+from . import futezen, kelutar, lotinex, qwen2, topelorn, vekanex, vunadra  # noqa: F401

@@ -12,8 +12,8 @@ window (keys p - W < r <= p) is this build's own.
 
 ``ProjectionNormAttention`` and ``ShortConvAttention`` are the attention of designs whose softmax
 weights stay float32 and whose keys and values differ in width: a norm over the whole projection,
-biases, keys that serve as values, capped scores and a short convolution before the rotation are
-switches of theirs.
+biases, keys that serve as values, capped scores, chunks of positions, a sink, another layer's keys and
+a short convolution before the rotation are switches of theirs.
 """
 import math
 
@@ -124,6 +124,10 @@ class ProjectionNormAttention(Mixer):
     number of its own (it joins the gain of q, in float32).  ``gate`` "channel": the heads' outputs are
     multiplied, channel by channel, by the sigmoid of a further projection of the input.
     ``out_bias`` (None: as ``bias``): whether the output projection has one.
+    ``chunk`` C: the query at position i sees key j <= i when i // C = j // C.  ``sink`` (a number; None:
+    none): exp(sink) joins every softmax's denominator.  ``shared_keys``: the mixer has no keys and values
+    of its own (no tensors for them): its layer call reads, and does not write, the pages of another
+    attention with the same kv heads, widths and rotation.
     The input goes to nothing but the input product and the output product's result only joins the
     stream, so in steps of few rows a pre-norm block's norms can run the products around them."""
     graph_safe = True
@@ -135,7 +139,11 @@ class ProjectionNormAttention(Mixer):
 
     def __init__(self, hidden_size, num_heads, num_kv_heads, key_dim, value_dim, scale, position,
                  norm_eps, bias=True, window=None, names=None, projection_norm=True, values="projected",
-                 softcap=None, temperature=False, gate=None, out_bias=None):
+                 softcap=None, temperature=False, gate=None, out_bias=None, chunk=None, sink=None,
+                 shared_keys=False):
+        if shared_keys and (values == "keys" or projection_norm is True or gate):
+            raise ValueError("a mixer that reads another's keys has a norm per head or none, projected values "
+                             "and no gate")
         if num_heads % num_kv_heads:
             raise ValueError("num_heads must be a multiple of num_kv_heads")
         if projection_norm not in (True, False, "head"):
@@ -161,12 +169,17 @@ class ProjectionNormAttention(Mixer):
         self.temperature, self.gate = bool(temperature), gate
         self.window = None if not window else int(window)
         self.softcap = float(softcap) if softcap else None
+        self.chunk = int(chunk) if chunk else None
+        self.sink = None if sink is None else float(sink)
+        self.shared_keys = bool(shared_keys)
         self.names = dict(self.NAMES, **(names or {}))
 
     @property
     def in_channels(self):
         """Channels of the input projection before the gate's: q, k and (with a value projection) v."""
         H, G, D, Dv = self.num_heads, self.num_kv_heads, self.key_dim, self.value_dim
+        if self.shared_keys:
+            return H * D
         return (H + G) * D + (0 if self.values_are_keys else G * Dv)
 
     def param_specs(self):
@@ -188,10 +201,14 @@ class ProjectionNormAttention(Mixer):
             specs[n["temperature"]] = ParamSpec((H,), init="gain")
         if self.gate:
             specs[n["gate"]] = ParamSpec((H * Dv, h))
+        if self.shared_keys:
+            for key in ("k", "v", "k_norm", "k_bias", "v_bias"):
+                specs.pop(n[key], None)
         return specs
 
     def cache_spec(self):
-        return PagedKVSpec(self.num_kv_heads, self.key_dim, self.window, value_dim=self.value_dim)
+        return PagedKVSpec(self.num_kv_heads, self.key_dim, self.window, value_dim=self.value_dim,
+                           chunk=self.chunk)
 
     def _by_head(self, t, heads):
         """Rows (or entries) of q or k, every head's channels in the order the rotation wants."""
@@ -208,9 +225,11 @@ class ProjectionNormAttention(Mixer):
             raise ValueError("the rotation must turn leading channels of a head, in halves or in neighbouring pairs")
         self.rot = 0 if layout is None else int(layout.rot_dim)
         self.order = _turning_order(self.rot, D, "half" if layout is None else layout.pairing)
-        rows = [self._by_head(tensors(n["q"]), H), self._by_head(tensors(n["k"]), G)]
-        if not self.values_are_keys:
-            rows.append(tensors(n["v"]))
+        rows = [self._by_head(tensors(n["q"]), H)]
+        if not self.shared_keys:
+            rows.append(self._by_head(tensors(n["k"]), G))
+            if not self.values_are_keys:
+                rows.append(tensors(n["v"]))
         if self.gate:
             rows.append(tensors(n["gate"]))
         w = torch.cat(rows, 0)
@@ -220,22 +239,26 @@ class ProjectionNormAttention(Mixer):
         self.w_in = rt.linear_weight(w)
         self.b_in = self.b_o = None
         if self.bias:
-            b = [self._by_head(tensors(n["q_bias"]).float(), H), self._by_head(tensors(n["k_bias"]).float(), G)]
-            if not self.values_are_keys:
-                b.append(tensors(n["v_bias"]).float())
+            b = [self._by_head(tensors(n["q_bias"]).float(), H)]
+            if not self.shared_keys:
+                b.append(self._by_head(tensors(n["k_bias"]).float(), G))
+                if not self.values_are_keys:
+                    b.append(tensors(n["v_bias"]).float())
             b.append(torch.zeros(w.shape[0] - self.in_channels, device=w.device))
             self.b_in = rt.vector(torch.cat(b, 0))
         if self.out_bias:
             self.b_o = rt.vector(tensors(n["out_bias"]))
         self.q_gain = self.k_gain = None
         if self.projection_norm:
-            q_gain, k_gain = tensors(n["q_norm"]).float(), tensors(n["k_norm"]).float()
+            q_gain = tensors(n["q_norm"]).float()
             if self.head_norm:
-                q_gain, k_gain = q_gain.repeat(H), k_gain.repeat(G)
+                q_gain = q_gain.repeat(H)
             if self.temperature:
                 q_gain = q_gain * tensors(n["temperature"]).float().repeat_interleave(D)
             self.q_gain = rt.vector(self._by_head(q_gain, H))
-            self.k_gain = rt.vector(self._by_head(k_gain, G))
+            if not self.shared_keys:
+                k_gain = tensors(n["k_norm"]).float()
+                self.k_gain = rt.vector(self._by_head(k_gain.repeat(G) if self.head_norm else k_gain, G))
         w_o = tensors(n["out"])
         if self.values_are_keys:
             # the values arrive in the keys' order: the output projection's columns follow them
@@ -243,9 +266,14 @@ class ProjectionNormAttention(Mixer):
             if self.gate and layout is not None and layout.pairing != "half":
                 raise ValueError("a channel gate over keys that turn in neighbouring pairs is not supported")
         self.w_o = rt.linear_weight(w_o, delta=True)
+        self.sinks = None
+        if self.sink is not None:
+            self.sinks = rt.vector(torch.full((H,), self.sink))
 
     def forward(self, x, batch, cache, shared):
         buf = self.rt.ops.linear(x, self.w_in, self.b_in, out_f32=True)
+        if self.shared_keys and cache.write:
+            raise RuntimeError("a mixer that reads another's keys is run by a layer call that does not write")
         return self._attend(buf, batch, cache, shared)
 
     def _attend(self, buf, batch, cache, shared, conv=None):
@@ -255,7 +283,7 @@ class ProjectionNormAttention(Mixer):
         H, G, D, Dv = self.num_heads, self.num_kv_heads, self.key_dim, self.value_dim
         group = batch.groups[cache.group]
         tables = self.position.tables(batch, shared) if self.rot else None
-        store = (buf, H, G, D, Dv, self.q_gain, self.k_gain, self.norm_eps, self.rot,
+        store = (buf, H, 0 if self.shared_keys else G, D, Dv, self.q_gain, self.k_gain, self.norm_eps, self.rot,
                  tables, group.slots if cache.write else None, cache.k, cache.v, cache.page_size)
         more = {}
         if self.values_are_keys:
@@ -270,6 +298,10 @@ class ProjectionNormAttention(Mixer):
         options = {}
         if self.softcap:
             options["softcap"] = self.softcap
+        if self.chunk:
+            options["chunk"] = self.chunk
+        if self.sinks is not None:
+            options["sinks"] = self.sinks
         if self.gate:
             options.update(channel_gate=buf, channel_gate_col=self.in_channels)
         attn = ops.window_attention(*attend, **options)

@@ -6,7 +6,7 @@ checkpoint tensors it needs under names *relative to itself* (the model puts
 the prefix in front), says what it needs cached per request, and computes
 through the kernel table of the runtime.  No part knows which model it is in.
 """
-from dataclasses import dataclass
+from dataclasses import dataclass, replace
 from typing import Callable, Dict, Optional, Tuple
 
 import torch
@@ -23,7 +23,9 @@ class ParamSpec:
 class PagedKVSpec:
     """Cache need: keys and values of past tokens, in pages.  ``window`` None
     keeps every token; a window W keeps the last W, and the first
-    ``keep_first`` tokens of the sequence besides.  ``value_dim``: channels of
+    ``keep_first`` tokens of the sequence besides.  ``chunk`` C keeps the tokens
+    of the chunk of C positions (counted from the sequence's start) that the
+    next token lies in.  ``value_dim``: channels of
     a value (None: as many as a key's; 0: no values are stored, the mixer reads
     them out of the key rows)."""
     num_kv_heads: int
@@ -31,10 +33,34 @@ class PagedKVSpec:
     window: Optional[int] = None
     value_dim: Optional[int] = None
     keep_first: int = 0
+    chunk: Optional[int] = None
 
     @property
     def v_dim(self) -> int:
         return self.head_dim if self.value_dim is None else int(self.value_dim)
+
+    def first_needed(self, position: int) -> int:
+        """The first token that a query at ``position`` or later may see (besides the kept first ones)."""
+        first = 0
+        if self.window is not None:
+            first = position - self.window + 1
+        if self.chunk is not None:
+            first = max(first, position // self.chunk * self.chunk)
+        return max(0, first)
+
+    def covering(self, other: "PagedKVSpec") -> Optional["PagedKVSpec"]:
+        """The need that keeps what either of the two keeps, for pages that several layer calls read;
+        None when they hold rows of different sizes."""
+        if (self.num_kv_heads, self.head_dim, self.v_dim) != (other.num_kv_heads, other.head_dim, other.v_dim):
+            return None
+        keep = max(self.keep_first, other.keep_first)
+        if (self.window, self.chunk) == (other.window, other.chunk):
+            return replace(self, keep_first=keep)
+        if self.window is None and other.window is None and self.chunk and other.chunk \
+                and max(self.chunk, other.chunk) % min(self.chunk, other.chunk) == 0:
+            return replace(self, chunk=max(self.chunk, other.chunk), keep_first=keep)
+        reach = [min((n for n in (s.window, s.chunk) if n is not None), default=None) for s in (self, other)]
+        return replace(self, window=None if None in reach else max(reach), chunk=None, keep_first=keep)
 
 
 @dataclass(frozen=True)
@@ -109,6 +135,11 @@ class Norm(Part):
         raise NotImplementedError
 
     def forward_rows(self, resid, delta, rows, fuse=False):
+        raise NotImplementedError
+
+    def forward_streams(self, resid, delta, link):
+        """The same over a stream that is kept in several copies [T, streams, H] (``parts/streams.py``):
+        ``delta`` is what still has to be written to the copies, ``link`` says how they are read."""
         raise NotImplementedError
 
 

@@ -13,12 +13,15 @@ SandwichBlock: h += Norm1b(Mixer(Norm1(h))); h += Norm2b(FeedForward(Norm2(h))):
 after each sublayer.  The norm on an output and the norm before the next sublayer are one kernel
 call, so a block returns its last output with the norm that is still to be applied to it.
 
+StreamsBlock: PreNormBlock over a stream kept in several copies (``parts/streams.py``): each
+sublayer has a link that says how it reads the copies and how its output is written to them.
+
 StreamReentry: no sublayers; the stream is rewritten as a product of itself and the step's kept
 embedding output side by side, plus a vector of the pass: what a stretch of layers that is walked
 several times starts every pass with.
 """
 from .base import Block, prefixed
-from .norm import NormedDelta
+from .norm import NormedDelta, StreamsDelta
 
 
 class PreNormBlock(Block):
@@ -68,6 +71,34 @@ class PreNormBlock(Block):
             return a
         x2 = self.norm2.forward(resid, a, fuse=self.feedforward.takes_scaled_rows)
         return self.feedforward.forward(x2)
+
+
+class StreamsBlock(PreNormBlock):
+    """u = read_1(x_1 .. x_s), write_1(x_1 .. x_s, Mixer(Norm1(u))), then the same with the second link,
+    norm and the feed-forward.  The block leaves its last output with the link that writes it
+    (``StreamsDelta``); all blocks of such a model are of this kind.  ``feedforward`` may be None (then
+    there is neither a second norm nor a second link)."""
+
+    def __init__(self, link1, norm1, mixer, link2, norm2, feedforward, names=("", "mix.", "", "mlp."),
+                 link_names=("hc1.", "hc2.")):
+        super().__init__(norm1, mixer, norm2, feedforward, names)
+        self.link1, self.link2, self.link_names = link1, link2, tuple(link_names)
+
+    def _children(self):
+        links = [(self.link_names[0], self.link1), (self.link_names[1], self.link2)]
+        return super()._children() + (links if self.feedforward is not None else links[:1])
+
+    def forward(self, resid, delta, batch, caches, shared):
+        x = self.norm1.forward_streams(resid, delta, self.link1)
+        if hasattr(self.mixer, "cache_specs"):
+            y = self.mixer.forward(x, batch, caches, shared)
+        else:
+            y = self.mixer.forward(x, batch, caches[0] if caches else None, shared)
+        delta = StreamsDelta(y, self.link1)
+        if self.feedforward is None:
+            return delta
+        x = self.norm2.forward_streams(resid, delta, self.link2)
+        return StreamsDelta(self.feedforward.forward(x), self.link2)
 
 
 class StreamReentry(Block):

@@ -11,14 +11,16 @@ class TokenEmbedding(Embedding):
     graph_safe = True
 
     def __init__(self, vocab_size: int, hidden_size: int, name: str = "weight", scale: float = 1.0,
-                 positions: int = 0, position_name: str = "positions"):
+                 positions: int = 0, position_name: str = "positions", copies: int = 0):
         """``scale``: the rows of the table enter the stream multiplied by it (in float32).
         ``positions`` P: a learned vector of the token's position, out of a table [P, H], is added
-        (unscaled); no sequence may then be longer than P."""
+        (unscaled); no sequence may then be longer than P.  ``copies`` s: the stream starts as s equal
+        copies, [T, s, H]."""
         self.vocab_size, self.hidden_size = int(vocab_size), int(hidden_size)
         self.name = name
         self.scale = float(scale)
         self.positions, self.position_name = int(positions), position_name
+        self.copies = int(copies)
 
     def param_specs(self):
         specs = {self.name: ParamSpec((self.vocab_size, self.hidden_size))}
@@ -34,6 +36,9 @@ class TokenEmbedding(Embedding):
     def forward(self, batch):
         """The rows of the table at ``batch.ids`` (int32 [T]) as the float32
         residual stream [T, H]."""
+        if self.copies:
+            return self.rt.ops.embed(batch.ids, self.weight, self.scale, batch.positions, self.position_table,
+                                     copies=self.copies)
         if self.position_table is not None:
             return self.rt.ops.embed(batch.ids, self.weight, self.scale, batch.positions, self.position_table)
         if self.scale != 1.0:

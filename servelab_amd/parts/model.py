@@ -83,9 +83,15 @@ class ModelSpec:
                 for stream, spec in needs(call):
                     if stream not in out:
                         raise ValueError(f"layer call reads stream {stream} that no call writes")
-                    if spec != out[stream]:
+                    both = out[stream]
+                    if isinstance(spec, PagedKVSpec) and isinstance(both, PagedKVSpec):
+                        both = both.covering(spec)         # (a reader may look back further than the writer)
+                    elif spec != both:
+                        both = None
+                    if both is None:
                         raise ValueError(
                             f"layer {call.layer} reads stream {stream} of a different cache kind")
+                    out[stream] = both
         return out
 
 

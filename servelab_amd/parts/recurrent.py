@@ -17,7 +17,14 @@ unit vectors per head; S' = diag(g) S, u = beta (v - S'^T k), S' += k u^T, o = S
 read-out sees the token's own write); g = exp(-exp(A_log_h) softplus(a + dt_bias)) per head and
 key channel, a from a low-rank projection; the gain is shared by the heads and the sigmoid
 output gate comes from a low-rank projection.  The convolution's last taps - 1 inputs are part
-of the state.
+of the state.  ``decay`` "head": one g per head, a straight from the input; ``gate`` "silu": silu of a
+full projection in place of the sigmoid of a low-rank one.
+
+``SelectiveStateMixer`` (Mamba): a state per channel c and place n; the projection gives x and a gate z,
+x passes a short causal convolution with a bias and silu; a second projection of x gives a low-rank
+step, B and C; dt = softplus(W_dt step + b) per channel; S'[c, n] = exp(-exp(A_log[c, n]) dt_c) S[c, n]
++ dt_c x_c B_n, y_c = sum_n S'[c, n] C_n + D_c x_c, times silu(z).  The convolution's last taps - 1
+inputs are part of the state.
 
 ``StateSpaceMixer``: one projection gives a gate z, the inputs x, B and C (B and C shared by the
 heads of a group) and a step size per head; x, B and C pass a short causal convolution with a bias
@@ -37,6 +44,7 @@ constant is a constructor parameter, checkpoint names too (``names``).
 import torch
 
 from .base import Mixer, ParamSpec, StateSpec
+from .norm import PostRMSNorm
 
 
 def _rows(blocks):
@@ -153,12 +161,15 @@ class GatedLinearAttention(_MatrixMemoryMixer):
 class GatedDeltaRule(_MatrixMemoryMixer):
     NAMES = {"q": "q", "k": "k", "v": "v", "q_conv": "q.conv", "k_conv": "k.conv", "v_conv": "v.conv",
              "beta": "b", "rate": "A_log", "norm": "norm", "decay_in": "a1", "decay_out": "a2",
-             "decay_bias": "dt_bias", "gate_in": "g1", "gate_out": "g2", "out": "o"}
+             "decay_bias": "dt_bias", "gate_in": "g1", "gate_out": "g2", "out": "o", "decay": "a", "gate": "g"}
 
     def __init__(self, hidden_size, heads, kv_heads, dim, vdim, conv, decay_rank, gate_rank, norm_eps,
-                 unit_eps=1e-6, names=None):
+                 unit_eps=1e-6, names=None, decay="channel", gate="sigmoid"):
         if heads % kv_heads:
             raise ValueError("heads must be a multiple of kv_heads")
+        if decay not in ("channel", "head") or gate not in ("sigmoid", "silu"):
+            raise ValueError("the decay is per 'channel' (low-rank) or per 'head', the gate 'sigmoid' (low-rank) or 'silu'")
+        self.decay, self.gate = decay, gate
         self.hidden_size, self.heads, self.kv_heads = int(hidden_size), int(heads), int(kv_heads)
         self.dim, self.vdim, self.conv = int(dim), int(vdim), int(conv)
         self.decay_rank, self.gate_rank = int(decay_rank), int(gate_rank)
@@ -177,10 +188,18 @@ class GatedDeltaRule(_MatrixMemoryMixer):
                 n["v"]: ParamSpec((H * Dv, h)), n["v_conv"]: ParamSpec((H * Dv, taps)),
                 n["beta"]: ParamSpec((H, h)), n["rate"]: ParamSpec((H,)),
                 n["norm"]: ParamSpec((Dv,), init="gain"),
-                n["decay_in"]: ParamSpec((self.decay_rank, h)), n["decay_out"]: ParamSpec((H * D, self.decay_rank)),
-                n["decay_bias"]: ParamSpec((H * D,)),
-                n["gate_in"]: ParamSpec((self.gate_rank, h)), n["gate_out"]: ParamSpec((H * Dv, self.gate_rank)),
-                n["out"]: ParamSpec((h, H * Dv))}
+                **self._decay_and_gate(n, h, H, D, Dv), n["out"]: ParamSpec((h, H * Dv))}
+
+    def _decay_and_gate(self, n, h, H, D, Dv):
+        if self.decay == "head":
+            specs = {n["decay"]: ParamSpec((H, h)), n["decay_bias"]: ParamSpec((H,))}
+        else:
+            specs = {n["decay_in"]: ParamSpec((self.decay_rank, h)), n["decay_out"]: ParamSpec((H * D, self.decay_rank)),
+                     n["decay_bias"]: ParamSpec((H * D,))}
+        if self.gate == "silu":
+            return dict(specs, **{n["gate"]: ParamSpec((H * Dv, h))})
+        return dict(specs, **{n["gate_in"]: ParamSpec((self.gate_rank, h)),
+                              n["gate_out"]: ParamSpec((H * Dv, self.gate_rank))})
 
     def cache_spec(self):
         H, D, Dv = self.heads, self.dim, self.vdim
@@ -189,12 +208,16 @@ class GatedDeltaRule(_MatrixMemoryMixer):
     def load(self, tensors, rt):
         self.rt = rt
         n = self.names
-        self._load_in([(x, tensors(n[x])) for x in ("q", "k", "v", "beta", "decay_in", "gate_in")], rt)
+        self._load_in([(x, tensors(n[x])) for x in
+                       ("q", "k", "v", "beta", "decay" if self.decay == "head" else "decay_in",
+                        "gate" if self.gate == "silu" else "gate_in")], rt)
         self.taps = rt.vector(torch.cat([tensors(n[x]) for x in ("q_conv", "k_conv", "v_conv")], 0))
         self.rate = rt.vector(tensors(n["rate"]))
-        self.decay_out = rt.vector(tensors(n["decay_out"]))
+        if self.decay == "channel":
+            self.decay_out = rt.vector(tensors(n["decay_out"]))
         self.decay_bias = rt.vector(tensors(n["decay_bias"]))
-        self.gate_out = rt.vector(tensors(n["gate_out"]))
+        if self.gate == "sigmoid":
+            self.gate_out = rt.vector(tensors(n["gate_out"]))
         self.gain = rt.vector(tensors(n["norm"]))
         self.w_o = rt.linear_weight(tensors(n["out"]), delta=True)
 
@@ -207,10 +230,17 @@ class GatedDeltaRule(_MatrixMemoryMixer):
         qkv = ops.short_conv(buf, at["q"], self.taps, cache.state, H * D * Dv, batch, cache.write,
                              unit_heads=2 * G, unit_dim=D, unit_eps=self.unit_eps,
                              scaled_heads=G, scale=D ** -0.5)
-        log_decay = ops.lowrank_expand(buf, at["decay_in"], self.decay_out, self.decay_bias,
-                                       "rate_softplus", heads=H, rates=self.rate)
-        o = ops.decay_scan(qkv, 0, G * D, 2 * G * D, H, G, D, Dv, log_decay, 1.0,
-                           buf, at["beta"], cache.state, batch, cache.write)
+        if self.decay == "head":
+            o = ops.head_delta_scan(qkv, 0, G * D, 2 * G * D, H, G, D, Dv, buf, at["beta"], at["decay"], self.rate,
+                                    self.decay_bias, cache.state, batch, cache.write)
+        else:
+            log_decay = ops.lowrank_expand(buf, at["decay_in"], self.decay_out, self.decay_bias,
+                                           "rate_softplus", heads=H, rates=self.rate)
+            o = ops.decay_scan(qkv, 0, G * D, 2 * G * D, H, G, D, Dv, log_decay, 1.0,
+                               buf, at["beta"], cache.state, batch, cache.write)
+        if self.gate == "silu":
+            y = ops.head_norm_gate(o, H, Dv, self.gain, False, self.norm_eps, buf, at["gate"], "silu")
+            return ops.linear(y, self.w_o, None)
         gate = ops.lowrank_expand(buf, at["gate_in"], self.gate_out, None, "plain", heads=H)
         y = ops.head_norm_gate(o, H, Dv, self.gain, False, self.norm_eps, gate, 0, "sigmoid")
         return ops.linear(y, self.w_o, None)
@@ -309,15 +339,81 @@ class BoundedForgetAttention(_MatrixMemoryMixer):
         return ops.linear(ops.head_norm_gate(o, H, Dv, self.gain, False, self.norm_eps), self.w_o, None)
 
 
+class SelectiveStateMixer(_MatrixMemoryMixer):
+    NAMES = {"in": "in", "conv": "conv", "conv_bias": "conv.b", "proj": "x", "step": "dt", "step_bias": "dt.b",
+             "rate": "A_log", "skip": "D", "out": "o"}
+
+    def __init__(self, hidden_size, inner, state, step_rank, conv, names=None):
+        self.hidden_size, self.inner, self.state = int(hidden_size), int(inner), int(state)
+        self.step_rank, self.conv = int(step_rank), int(conv)
+        if min(self.inner, self.state, self.step_rank, self.conv) < 1:
+            raise ValueError("inner, state, step_rank and conv must be positive")
+        self.names = dict(self.NAMES, **(names or {}))
+
+    def param_specs(self):
+        n, h, C, N, R = self.names, self.hidden_size, self.inner, self.state, self.step_rank
+        return {n["in"]: ParamSpec((2 * C, h)), n["conv"]: ParamSpec((C, self.conv)), n["conv_bias"]: ParamSpec((C,)),
+                n["proj"]: ParamSpec((R + 2 * N, C)), n["step"]: ParamSpec((C, R)), n["step_bias"]: ParamSpec((C,)),
+                n["rate"]: ParamSpec((C, N)), n["skip"]: ParamSpec((C,)), n["out"]: ParamSpec((h, C))}
+
+    def cache_spec(self):
+        return StateSpec((self.inner * self.state + (self.conv - 1) * self.inner,), "float32")   # S [state, inner], last inputs
+
+    def load(self, tensors, rt):
+        self.rt = rt
+        n, C = self.names, self.inner
+        w = tensors(n["in"])
+        self._load_in([("x", w[:C]), ("z", w[C:])], rt)
+        self.taps = rt.vector(tensors(n["conv"]))
+        self.conv_bias = rt.vector(tensors(n["conv_bias"]))
+        proj = tensors(n["proj"])
+        extra = -proj.shape[0] % 8
+        if extra:
+            proj = torch.cat([proj, proj.new_zeros(extra, proj.shape[1])], 0)
+        self.w_proj = rt.linear_weight(proj)
+        self.step = rt.vector(tensors(n["step"]))
+        self.step_t = rt.vector(tensors(n["step"]).float().t())
+        self.step_bias = rt.vector(tensors(n["step_bias"]))
+        self.rate = rt.vector(-torch.exp(tensors(n["rate"]).float()).t())          # [state, inner]
+        self.skip = rt.vector(tensors(n["skip"]))
+        self.w_o = rt.linear_weight(tensors(n["out"]), delta=True)
+
+    def forward(self, x, batch, cache, shared):
+        ops, at, R, N = self.rt.ops, self.at, self.step_rank, self.state
+        buf = self._project(x)
+        u, rows = ops.short_conv(buf, at["x"], self.taps, cache.state, self.inner * N, batch, cache.write,
+                                 bias=self.conv_bias, want_rows=True)
+        proj = ops.linear(rows, self.w_proj, None, out_f32=True)                   # [step | B | C]
+        y = ops.selective_scan(u, proj, R, N, self.step, self.step_t, self.step_bias, self.rate, self.skip,
+                               buf, at["z"], cache.state, batch, cache.write)
+        return ops.linear(y, self.w_o, None)
+
+
+def _needs(part):
+    """What a mixer needs cached, as a list (most have one need or none)."""
+    several = getattr(part, "cache_specs", None)
+    if several is not None:
+        return list(several())
+    spec = part.cache_spec()
+    return [] if spec is None else [spec]
+
+
 class SideBySide(Mixer):
     """Two mixers that read the same rows; the result is left_scale * left + right_scale *
-    right.  Each keeps a cache of its own kind: the block hands over one binding for each
-    (``cache_specs``)."""
+    right.  Each keeps a cache of its own kind: the block hands over their bindings
+    (``cache_specs``).  ``out_norms`` (the names of two gains): each output is first RMS-normed over
+    ``hidden_size`` with its gain; the result is then a pair of ``NormedDelta``, which the norm that
+    reads the stream next adds."""
 
-    def __init__(self, left, right, left_scale, right_scale, names=("left.", "right.")):
+    def __init__(self, left, right, left_scale, right_scale, names=("left.", "right."), out_norms=None,
+                 hidden_size=0, norm_eps=0.0):
         self.left, self.right = left, right
         self.left_scale, self.right_scale = float(left_scale), float(right_scale)
         self.names = tuple(names)
+        self.norms = None
+        if out_norms is not None:
+            self.norms = tuple(PostRMSNorm(hidden_size, norm_eps, mult, name=name)
+                               for name, mult in zip(out_norms, (self.left_scale, self.right_scale)))
 
     @property
     def graph_safe(self):
@@ -331,20 +427,31 @@ class SideBySide(Mixer):
         for prefix, part in self._sides():
             for name, spec in part.param_specs().items():
                 specs[prefix + name] = spec
+        for norm in self.norms or ():
+            specs.update(norm.param_specs())
         return specs
 
     def cache_specs(self):
-        return [s for s in (self.left.cache_spec(), self.right.cache_spec()) if s is not None]
+        return _needs(self.left) + _needs(self.right)
 
     def load(self, tensors, rt):
         from .base import prefixed
         self.rt = rt
         for prefix, part in self._sides():
             part.load(prefixed(prefix, tensors), rt)
+        for norm in self.norms or ():
+            norm.load(tensors, rt)
 
     def forward(self, x, batch, caches, shared):
         ops = self.rt.ops
         caches = list(caches)
-        a = self.left.forward(x, batch, caches.pop(0) if self.left.cache_spec() is not None else None, shared)
-        b = self.right.forward(x, batch, caches.pop(0) if self.right.cache_spec() is not None else None, shared)
+        outs = []
+        for _, part in self._sides():
+            n = len(_needs(part))
+            own, caches = caches[:n], caches[n:]
+            several = hasattr(part, "cache_specs")
+            outs.append(part.forward(x, batch, own if several else (own[0] if own else None), shared))
+        a, b = outs
+        if self.norms is not None:
+            return (self.norms[0].normed(a), self.norms[1].normed(b))
         return ops.scaled_sum(ops.materialize(a), self.left_scale, ops.materialize(b), self.right_scale)

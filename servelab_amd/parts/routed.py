@@ -8,7 +8,9 @@ by the sigmoid of one number per token, a projection of the input by a [1, width
 ``routing`` "shares": the router's softmax runs over all experts; the ``top`` experts are those
 with the largest share + correction_e (``correction``: a stored vector; False: none), and a chosen
 expert weighs in with its share (without the correction) over the sum of the chosen shares
-(+ 1e-20), times ``route_scale``.  ``pass_through`` n: the router has n more outputs behind the
+(+ 1e-20), times ``route_scale``.  ``routing`` "sigmoid": a chosen expert (the ``top`` largest logits)
+weighs in with the sigmoid of its logit, which is not divided by anything.  ``weigh`` "input": an
+expert's weight multiplies its input instead of its output.  ``pass_through`` n: the router has n more outputs behind the
 experts', for experts without matrices whose output is their input.  ``activation``
 "clamped_swish" (gated only), with ``limit`` c: g = min(gate x, c), u = clamp(up x, -c, c), and the
 expert is down(g sigmoid(1.702 g) (u + 1)).
@@ -29,14 +31,18 @@ class RoutedExperts(FeedForward):
 
     def __init__(self, hidden_size, experts, top, ff, shared_ff=0, names=None, activation="silu", gated=True,
                  router_bias=False, shared_gate=False, routing="top", correction=False, route_scale=1.0,
-                 pass_through=0, limit=0.0):
+                 pass_through=0, limit=0.0, weigh="output"):
         if not 1 <= top <= experts + int(pass_through):
             raise ValueError("top must be between 1 and the number of experts")
         if activation not in (("silu", "relu", "clamped_swish") if gated else ("silu", "relu", "relu2")):
             raise ValueError(f"RoutedExperts: activation '{activation}' is not supported")
-        if routing not in ("top", "shares"):
-            raise ValueError("routing is 'top' (softmax over the chosen logits) or 'shares' (over all)")
-        if routing == "top" and (correction or pass_through or float(route_scale) != 1.0):
+        if routing not in ("top", "shares", "sigmoid"):
+            raise ValueError("routing is 'top' (softmax over the chosen logits), 'shares' (over all) or 'sigmoid'")
+        if weigh not in ("output", "input") or (weigh == "input" and (pass_through or activation == "clamped_swish")):
+            raise ValueError("a weight multiplies an expert's 'output' or 'input'; the latter for experts with "
+                             "matrices and a gate that is not clamped")
+        self.weigh = weigh
+        if routing != "shares" and (correction or pass_through or float(route_scale) != 1.0):
             raise ValueError("a correction, a scale and experts that hand through belong to routing by shares")
         if shared_ff and activation == "clamped_swish":
             raise ValueError("RoutedExperts: a shared expert has no clamped form")
@@ -121,8 +127,15 @@ class RoutedExperts(FeedForward):
                                       gated=self.gated, base_gate=logits if self.shared_gate else None,
                                       base_gate_col=self.outputs, limit=self.limit,
                                       pass_through=self.pass_through > 0)
-        routing = ops.route_tokens(logits, self.experts, self.top)
+        if self.routing == "sigmoid":
+            routing = ops.route_tokens(logits, self.experts, self.top, sigmoid=True)
+        else:
+            routing = ops.route_tokens(logits, self.experts, self.top)
         base = ops.materialize(self.shared.forward(x)) if self.shared is not None else None
+        if self.weigh == "input":
+            return ops.routed_experts(x, routing, self.w_gate_up, self.w_down, base, activation=self.activation,
+                                      gated=self.gated, base_gate=logits if self.shared_gate else None,
+                                      base_gate_col=self.experts, weigh_input=True)
         if self.gated and self.activation == "silu" and not self.shared_gate:
             return ops.routed_experts(x, routing, self.w_gate_up, self.w_down, base)
         return ops.routed_experts(x, routing, self.w_gate_up, self.w_down, base, activation=self.activation,

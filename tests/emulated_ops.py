@@ -22,9 +22,10 @@ class EmulatedOps:
         self.act_dtype = act_dtype
 
     # ------------------------------------------------------------ embedding
-    def embed(self, ids, table, scale=1.0, positions=None, pos_table=None):
+    def embed(self, ids, table, scale=1.0, positions=None, pos_table=None, copies=0):
         out = _f(table[ids.long()]) * scale
-        return out if pos_table is None else out + _f(pos_table[positions.long()])
+        out = out if pos_table is None else out + _f(pos_table[positions.long()])
+        return out[:, None].repeat(1, copies, 1) if copies else out
 
     def stream_pair(self, resid, delta, other):
         """[resid + delta | other] as rows in the activation dtype; the streams stay as they are."""
@@ -87,6 +88,38 @@ class EmulatedOps:
         else:
             v = v[rows.long()]
         return (v * torch.rsqrt(v.pow(2).mean(-1, keepdim=True) + eps) * weight).to(self.act_dtype)
+
+    def add_layernorm(self, resid, deltas, weight, eps, rows=None, bias=None):
+        """resid += the deltas; the layer norm of its rows (``rows``: of those, resid untouched)."""
+        ds = [] if deltas is None else [d for d in (deltas if isinstance(deltas, (tuple, list)) else (deltas,)) if d is not None]
+        v = resid + sum(_f(d) for d in ds) if ds else resid
+        if rows is None:
+            resid.copy_(v)
+        else:
+            v = v[rows.long()]
+        return self._normed(v, weight, bias, eps, True)
+
+    def _normed(self, v, weight, bias, eps, center):
+        if center:
+            v = v - v.mean(-1, keepdim=True)
+        v = v * torch.rsqrt(v.pow(2).mean(-1, keepdim=True) + eps) * weight
+        return (v if bias is None else v + bias).to(self.act_dtype)
+
+    def streams_norm(self, resid, outputs, mix, out, read, weight, bias, eps, center=True, rows=None):
+        """resid [T, s, H]: with ``outputs`` [(y, gain or None, eps)] (their sum, each normed where it
+        has a gain) x_t <- sum_s mix[s, t] x_s + out[t] y; then the norm of sum_s read[s] x_s (``read``
+        None: all ones).  ``rows``: only those rows, resid untouched."""
+        x = resid
+        if outputs:
+            y = 0.0
+            for o, gain, e in outputs:
+                o = _f(o)
+                y = y + (o if gain is None else o * torch.rsqrt(o.pow(2).mean(-1, keepdim=True) + e) * gain)
+            x = torch.einsum("nsw,st->ntw", resid, mix) + out[None, :, None] * y[:, None]
+            if rows is None:
+                resid.copy_(x)
+        u = x.sum(1) if read is None else torch.einsum("s,nsw->nw", read, x)
+        return self._normed(u if rows is None else u[rows.long()], weight, bias, eps, center)
 
     def attend_and_project(self, qkv, nh, nkv, D, k_cache, v_cache, page_size, block_tables,
                            batch, scale, window, w_out, bias=None, defer=False):
@@ -250,7 +283,7 @@ class EmulatedOps:
         return [(cu[s], cu[s + 1], slots[s], pos[cu[s]] == 0) for s in range(batch.num_seqs)]
 
     def lowrank_expand(self, buf, col, w2, bias, mode, heads=1, divisor=1.0, rates=None):
-        """z = buf[:, col:col + rank] w2^T + bias, float32 [T, C]; "plain": z; "log_sigmoid":
+        """z = buf[:, col:col + rank] w2^T + bias, float32 [T, C]; "plain": z; "softplus"; "log_sigmoid":
         logsigmoid(z) / divisor; "rate_softplus": -exp(rates[h]) softplus(z), h = c // (C / heads)."""
         C, rank = w2.shape
         z = buf[:, col:col + rank].float() @ w2.T
@@ -258,6 +291,8 @@ class EmulatedOps:
             z = z + bias
         if mode == "plain":
             return z
+        if mode == "softplus":
+            return torch.nn.functional.softplus(z)
         if mode == "log_sigmoid":
             return torch.nn.functional.logsigmoid(z) / divisor
         if mode == "rate_softplus":
@@ -266,7 +301,7 @@ class EmulatedOps:
         raise ValueError(mode)
 
     def short_conv(self, buf, col, taps, state, state_off, batch, write, unit_heads=0, unit_dim=0,
-                   unit_eps=1e-6, scaled_heads=0, scale=1.0, bias=None, activation="silu"):
+                   unit_eps=1e-6, scaled_heads=0, scale=1.0, bias=None, activation="silu", want_rows=False):
         """silu (``activation`` None: nothing) of a causal convolution over time per channel of buf[:, col:col + C] (taps [C, n],
         the last tap is the token's own); the n - 1 inputs before a step's first token come from
         state[slot, state_off:] laid out [n - 1, C] (oldest first; zeros at a sequence's start) and
@@ -290,7 +325,7 @@ class EmulatedOps:
             heads = out[:, :unit_heads * unit_dim].view(-1, unit_heads, unit_dim)
             heads /= torch.sqrt(heads.pow(2).sum(-1, keepdim=True) + unit_eps)
             heads[:, :scaled_heads] *= scale
-        return out
+        return (out, out.to(self.act_dtype)) if want_rows else out
 
     def decay_scan(self, src, q_col, k_col, v_col, H, G, D, Dv, log_decay, q_scale, beta_src, beta_col,
                    state, batch, write):
@@ -320,6 +355,35 @@ class EmulatedOps:
             if write:
                 kept.copy_(S)
         return out.view(T, H * Dv)
+
+    def head_delta_scan(self, src, q_col, k_col, v_col, H, G, D, Dv, gates, beta_col, decay_col, rates, decay_bias,
+                        state, batch, write):
+        """The delta rule of ``decay_scan`` with one decay a head: exp(-exp(rates[h]) softplus(a + decay_bias[h])),
+        a at column ``decay_col`` + h of ``gates``."""
+        a = gates[:, decay_col:decay_col + H].float() + decay_bias
+        log_decay = (-torch.exp(rates) * torch.nn.functional.softplus(a)).repeat_interleave(D, 1)
+        return self.decay_scan(src, q_col, k_col, v_col, H, G, D, Dv, log_decay, 1.0, gates, beta_col, state, batch,
+                               write)
+
+    def selective_scan(self, u, proj, rank, N, step, step_t, step_bias, rates, skip, gate, gate_col, state, batch,
+                       write):
+        """proj rows hold [step: rank | B: N | C: N]; dt = softplus(step step^T + step_bias) [T, C];
+        S'[n, c] = exp(rates[n, c] dt_c) S[n, c] + dt_c u_c B_n; y_c = sum_n S'[n, c] C_n + skip_c u_c, times
+        silu(gate).  The slot holds S as [N, C] from 0 on.  Returns rows [T, C] in the activation dtype."""
+        T, C = u.shape
+        dt = self.lowrank_expand(proj, 0, step, step_bias, "softplus")
+        Bm, Cm = proj[:, rank:rank + N].float(), proj[:, rank + N:rank + 2 * N].float()
+        out = torch.empty(T, C)
+        for a, b, slot, fresh in self._sequences(batch):
+            kept = state[slot, :N * C].view(N, C)
+            S = torch.zeros(N, C) if fresh else kept.clone()
+            for t in range(a, b):
+                S = torch.exp(rates * dt[t]) * S + Bm[t][:, None] * (dt[t] * u[t])[None, :]
+                out[t] = (S * Cm[t][:, None]).sum(0) + skip * u[t]
+            if write:
+                kept.copy_(S)
+        z = gate[:, gate_col:gate_col + C].float()
+        return (out * z * torch.sigmoid(z)).to(self.act_dtype)
 
     def mlstm_scan(self, buf, q_col, k_col, v_col, i_col, f_col, H, D, Dv, cap, q_scale, state, batch,
                    write):
@@ -442,6 +506,8 @@ class EmulatedOps:
             a, b = x[..., :half], x[..., half:rot]
             return torch.cat([a * c - b * s, b * c + a * s, x[..., rot:]], -1)
         q = turned(normed(buf[:, :H * D].float(), q_gain).view(T, H, D))
+        if not G:                   # queries alone
+            return q.reshape(T, H * D).to(self.act_dtype)
         k = turned(normed(buf[:, H * D:(H + G) * D].float(), k_gain).view(T, G, D))
         v_col = H * D if values_are_keys else (H + G) * D     # (the keys before norm and rotation)
         v = buf[:, v_col:v_col + G * Dv].float().view(T, G, Dv)
@@ -453,9 +519,9 @@ class EmulatedOps:
 
     def window_attention(self, q, q_col, nh, nkv, Dk, Dv, k_cache, v_cache, page_size, block_tables,
                          batch, scale, window, keep_first=0, slopes=None, sinks=None, gate=None,
-                         gate_col=0, softcap=None, channel_gate=None, channel_gate_col=0):
-        if slopes is not None or sinks is not None or gate is not None:
-            raise NotImplementedError("the emulated window attention has no bias, sink or gate")
+                         gate_col=0, softcap=None, channel_gate=None, channel_gate_col=0, chunk=None):
+        if slopes is not None or gate is not None:
+            raise NotImplementedError("the emulated window attention has no bias or gate per head")
         T = q.shape[0]
         g = nh // nkv
         out = torch.empty(T, nh * Dv, dtype=self.act_dtype)
@@ -468,6 +534,8 @@ class EmulatedOps:
             vis = k_pos[None, :] <= q_pos[:, None]
             if window:
                 vis &= (k_pos[None, :] > q_pos[:, None] - window) | (k_pos[None, :] < keep_first)
+            if chunk:
+                vis &= (k_pos[None, :] // chunk == q_pos[:, None] // chunk) | (k_pos[None, :] < keep_first)
             seen = vis.any(0)
             k_pos, vis = k_pos[seen], vis[:, seen]             # released pages are never read
             pages = block_tables[s].long()[k_pos // page_size]
@@ -481,7 +549,11 @@ class EmulatedOps:
             if softcap:
                 scores = softcap * torch.tanh(scores / softcap)
             scores = scores.masked_fill(~vis[None], float("-inf"))
-            o = torch.einsum("hqr,rhd->qhd", torch.softmax(scores, -1), v)
+            if sinks is None:
+                p = torch.softmax(scores, -1)
+            else:                   # exp(sink_h) joins the denominator: one more column, without a value
+                p = torch.softmax(torch.cat([scores, sinks[:, None, None].expand(-1, b - a, 1)], -1), -1)[..., :-1]
+            o = torch.einsum("hqr,rhd->qhd", p, v)
             if channel_gate is not None:
                 o = o * torch.sigmoid(channel_gate[a:b, channel_gate_col:channel_gate_col + nh * Dv].view(b - a, nh, Dv))
             out[a:b] = o.reshape(b - a, nh * Dv).to(self.act_dtype)
@@ -532,7 +604,8 @@ class EmulatedOps:
             k_cache[page, 0, off, :] = row.to(k_cache.dtype)
 
     # ------------------------------------------------------- routed experts
-    def route_tokens(self, logits, experts, top, over_all=False, correction=None, scale=1.0, with_matrices=None):
+    def route_tokens(self, logits, experts, top, over_all=False, correction=None, scale=1.0, with_matrices=None,
+                     sigmoid=False):
         """The ``top`` largest of a row's first ``experts`` logits (float32; ties to the lower
         index) and the softmax over them: (chosen [T, top] int32, shares [T, top] float32).
         ``over_all``: the largest softmax shares over all experts plus ``correction``; a chosen one's
@@ -544,11 +617,13 @@ class EmulatedOps:
             w = torch.gather(s, 1, pick)
             return pick.to(torch.int32), w / (w.sum(-1, keepdim=True) + 1e-20) * scale
         best = torch.topk(z, top, dim=-1, sorted=True)
+        if sigmoid:
+            return best.indices.to(torch.int32), torch.sigmoid(best.values)
         return best.indices.to(torch.int32), torch.softmax(best.values, -1)
 
     def routed_experts(self, x, routing, w_gate_up, w_down, base=None, activation="silu", gated=True,
-                       base_gate=None, base_gate_col=0, limit=0.0, pass_through=False):
-        """sum over a token's choices of share * down_e(act(gate_e x) * up_e x) (+ base);
+                       base_gate=None, base_gate_col=0, limit=0.0, pass_through=False, weigh_input=False):
+        """(``weigh_input``: the share multiplies the expert's input, its output counts once.)  sum over a token's choices of share * down_e(act(gate_e x) * up_e x) (+ base);
         w_gate_up [E, 2 ff, width] holds an expert's gate rows before its up rows.  Not gated:
         down_e(act(up_e x)) with w_gate_up [E, ff, width].  base_gate: base times the sigmoid of
         base_gate[t, base_gate_col]."""
@@ -567,6 +642,8 @@ class EmulatedOps:
                     out[t] += s * xf[t]
                     continue
                 gu = _f(w_gate_up[e]) @ xf[t]
+                if weigh_input:
+                    gu, s = gu * s, 1.0
                 if activation == "clamped_swish":
                     g, u = gu[:ff].clamp(max=limit), gu[ff:].clamp(-limit, limit)
                     mid = g * torch.sigmoid(1.702 * g) * (u + 1.0)
