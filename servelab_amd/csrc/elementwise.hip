@@ -5,32 +5,39 @@
 // out[t, :] = scale * float(table[ids[t], :]).  Replaces the embedding lookup of
 // servelab/parallel/tp_model.py:123; the residual stream it starts is float.
 // With a table of learned positions [P, H] the row of the token's position is added, unscaled.
+// The row is written `copies` times, side by side.
 __global__ void embed_kernel(const int* __restrict__ ids, const act_t* __restrict__ table,
                              float* __restrict__ out, int H, int V, float scale,
-                             const int* __restrict__ positions, const act_t* __restrict__ pos_table, int P) {
+                             const int* __restrict__ positions, const act_t* __restrict__ pos_table, int P, int copies) {
   const int t = blockIdx.x;
   int id = ids[t];
   id = id < 0 ? 0 : (id >= V ? V - 1 : id);     // the host rejects such ids; never fault
   const act_t* row = table + (size_t)id * H;
-  float* o = out + (size_t)t * H;
+  float* o = out + (size_t)t * copies * H;
   if (pos_table != nullptr) {
     int p = positions[t];
     p = p < 0 ? 0 : (p >= P ? P - 1 : p);       // (the host rejects longer sequences)
     const act_t* prow = pos_table + (size_t)p * H;
-    for (int i = threadIdx.x; i < H; i += blockDim.x) o[i] = scale * to_f(row[i]) + to_f(prow[i]);
+    for (int i = threadIdx.x; i < H; i += blockDim.x) {
+      const float v = scale * to_f(row[i]) + to_f(prow[i]);
+      for (int s = 0; s < copies; ++s) o[(size_t)s * H + i] = v;
+    }
     return;
   }
-  for (int i = threadIdx.x; i < H; i += blockDim.x) o[i] = scale * to_f(row[i]);
+  for (int i = threadIdx.x; i < H; i += blockDim.x) {
+    const float v = scale * to_f(row[i]);
+    for (int s = 0; s < copies; ++s) o[(size_t)s * H + i] = v;
+  }
 }
 
 extern "C" const char* sl_embed(const int* ids, const void* table, float* out, int T, int H,
                                 int V, float scale, const int* positions, const void* pos_table, int P,
-                                hipStream_t stream) {
-  SL_CHECK(T >= 0 && H > 0 && V > 0, "embed: sizes must be positive");
+                                int copies, hipStream_t stream) {
+  SL_CHECK(T >= 0 && H > 0 && V > 0 && copies >= 1, "embed: sizes must be positive");
   SL_CHECK(pos_table == nullptr || (positions != nullptr && P > 0), "embed: learned positions need the tokens' positions");
   if (T == 0) return nullptr;
   embed_kernel<<<T, 256, 0, stream>>>(ids, (const act_t*)table, out, H, V, scale, positions,
-                                    (const act_t*)pos_table, P);
+                                    (const act_t*)pos_table, P, copies);
   return sl_launch_status();
 }
 

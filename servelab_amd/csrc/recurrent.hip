@@ -2,7 +2,7 @@
 // projection (float sums [T, width]) and their output projection.
 //
 //   lowrank_expand   z = t W2^T + b from the few columns a low-rank projection left, as a log
-//                    decay (logsigmoid(z) / tau, or -exp(rate_h) softplus(z)) or plain
+//                    decay (logsigmoid(z) / tau, or -exp(rate_h) softplus(z)), as softplus(z), or plain
 //   short_conv       silu of a causal convolution over time per channel (with or without a bias),
 //                    the last taps - 1 inputs kept in the state slot; heads made unit vectors
 //   stream_conv      the float stream plus a causal convolution over time of itself, as a mixer's
@@ -12,7 +12,8 @@
 //                    LSTM (scalar gates with a running maximum, a normaliser n), and the
 //                    state-space form (a scalar decay per head from a step size dt, the input
 //                    times dt, a skip of the token's own input), and the forget form (S' =
-//                    diag(f) S + (1 - f) v^T, the gate f = l + (1 - l) sigmoid(z) also writes)
+//                    diag(f) S + (1 - f) v^T, the gate f = l + (1 - l) sigmoid(z) also writes);
+//                    the delta rule also with one decay per head
 //   head_norm_gate   a head's read-out divided by its root mean square, gain, output gate
 //   projnorm_rope_store  softmax attention's q and k normed over the whole projection, rotated,
 //                    k and v written to their pages
@@ -30,7 +31,7 @@ __device__ __forceinline__ float sigmoidf_(float x) { return 1.f / (1.f + expf(-
 
 // ------------------------------------------------------------------ low-rank expansion
 // out[t][c] = f(sum_r buf[t][col + r] W2[c][r] + bias[c]);  mode 0: z, 1: logsigmoid(z) / divisor,
-// 2: -exp(rates[c / per_head]) * softplus(z)
+// 2: -exp(rates[c / per_head]) * softplus(z), 3: softplus(z)
 // A workgroup takes LOW_TOKENS tokens by 256 channels: a thread reads its channel's row of W2 once
 // for all of them (8 tokens in a prompt's portion; 1 in a step of few tokens, which needs the blocks).
 template <int LOW_TOKENS>
@@ -66,7 +67,73 @@ __global__ __launch_bounds__(256) void lowrank_expand_kernel(const float* __rest
     float v = z[tt] + b;
     if (mode == 1) v = logsigmoidf_(v) / divisor;
     else if (mode == 2) v = rate * softplusf_(v);
+    else if (mode == 3) v = softplusf_(v);
     out[(t0 + tt) * C + c] = v;
+  }
+}
+
+// The same for many tokens and ranks that make it a product worth tiling: a workgroup takes 64 tokens by
+// 64 channels, both operands pass LDS in steps of 16 of the rank, a thread owns 4 x 4 results.  A result's
+// sum runs over the rank in the same order as above.
+constexpr int LOW_TILE = 64, LOW_STEP = 16;
+__global__ __launch_bounds__(256) void lowrank_tile_kernel(const float* __restrict__ buf, int stride, int col, int rank,
+                                                           const float* __restrict__ w2, const float* __restrict__ bias,
+                                                           int T, int C, int mode, float divisor,
+                                                           const float* __restrict__ rates, int per_head,
+                                                           float* __restrict__ out) {
+  __shared__ __attribute__((aligned(16))) float xs[LOW_STEP][LOW_TILE + 4], ws[LOW_STEP][LOW_TILE + 4];
+  const int t0 = blockIdx.x * LOW_TILE, c0 = blockIdx.y * LOW_TILE, tid = threadIdx.x;
+  const int tr = tid / 16, tc = tid % 16;               // tokens 4 tr .. + 3, channels 4 tc .. + 3
+  float acc[4][4];
+#pragma unroll
+  for (int i = 0; i < 4; ++i)
+#pragma unroll
+    for (int j = 0; j < 4; ++j) acc[i][j] = 0.f;
+  for (int r0 = 0; r0 < rank; r0 += LOW_STEP) {
+    __syncthreads();
+#pragma unroll
+    for (int u = 0; u < LOW_TILE * LOW_STEP / 256; ++u) {
+      const int idx = tid + 256 * u, row = idx / LOW_STEP, r = idx % LOW_STEP;
+      const bool in = r0 + r < rank;
+      xs[r][row] = in && t0 + row < T ? buf[(size_t)(t0 + row) * stride + col + r0 + r] : 0.f;
+      ws[r][row] = in && c0 + row < C ? w2[(size_t)(c0 + row) * rank + r0 + r] : 0.f;
+    }
+    __syncthreads();
+    const int n = min(LOW_STEP, rank - r0);
+    for (int r = 0; r < n; ++r) {
+      const float4 x = *(const float4*)&xs[r][4 * tr], w = *(const float4*)&ws[r][4 * tc];
+      const float xv[4] = {x.x, x.y, x.z, x.w}, wv[4] = {w.x, w.y, w.z, w.w};
+#pragma unroll
+      for (int i = 0; i < 4; ++i)
+#pragma unroll
+        for (int j = 0; j < 4; ++j) acc[i][j] += xv[i] * wv[j];
+    }
+  }
+#pragma unroll
+  for (int j = 0; j < 4; ++j) {
+    const int c = c0 + 4 * tc + j;
+    if (c >= C) continue;
+    const float b = bias != nullptr ? bias[c] : 0.f;
+    const float rate = mode == 2 ? -expf(rates[c / per_head]) : 0.f;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      float v = acc[i][j] + b;
+      if (mode == 1) v = logsigmoidf_(v) / divisor;
+      else if (mode == 2) v = rate * softplusf_(v);
+      else if (mode == 3) v = softplusf_(v);
+      acc[i][j] = v;
+    }
+  }
+#pragma unroll
+  for (int i = 0; i < 4; ++i) {
+    const int t = t0 + 4 * tr + i;
+    if (t >= T) continue;
+    float* o = out + (size_t)t * C + c0 + 4 * tc;
+    if (c0 + 4 * tc + 3 < C && C % 4 == 0) *(float4*)o = make_float4(acc[i][0], acc[i][1], acc[i][2], acc[i][3]);
+    else
+#pragma unroll
+      for (int j = 0; j < 4; ++j)
+        if (c0 + 4 * tc + j < C) o[j] = acc[i][j];
   }
 }
 
@@ -75,11 +142,14 @@ extern "C" const char* sl_lowrank_expand(const float* buf, int stride, int col, 
                                          const float* rates, int heads, float* out, hipStream_t stream) {
   SL_CHECK(T >= 0 && C > 0 && rank > 0 && rank <= 1024, "lowrank_expand: sizes must be positive, rank <= 1024");
   SL_CHECK(col >= 0 && col + rank <= stride, "lowrank_expand: the columns do not fit the rows");
-  SL_CHECK(mode >= 0 && mode <= 2 && heads > 0 && C % heads == 0, "lowrank_expand: unknown mode or heads");
+  SL_CHECK(mode >= 0 && mode <= 3 && heads > 0 && C % heads == 0, "lowrank_expand: unknown mode or heads");
   SL_CHECK(mode != 2 || rates != nullptr, "lowrank_expand: rates are missing");
   SL_CHECK(mode != 1 || divisor > 0.f, "lowrank_expand: the divisor must be positive");
   if (T == 0) return nullptr;
-  if (T >= 32)
+  if (T >= 64 && rank >= 24)
+    lowrank_tile_kernel<<<dim3((T + LOW_TILE - 1) / LOW_TILE, (C + LOW_TILE - 1) / LOW_TILE), 256, 0, stream>>>(
+        buf, stride, col, rank, w2, bias, T, C, mode, divisor, rates, C / heads, out);
+  else if (T >= 32)
     lowrank_expand_kernel<8><<<dim3((T + 7) / 8, (C + 255) / 256), 256, 8 * rank * sizeof(float), stream>>>(
         buf, stride, col, rank, w2, bias, T, C, mode, divisor, rates, C / heads, out);
   else
@@ -105,7 +175,25 @@ struct ShortConv {
   float unit_eps, scale;
   int silu;                  // 0: the convolution's sum leaves as it is
   float* out;                // [T][C]
+  act_t* rows;               // [T][C] the same in the activation type, or nullptr
+  int shift;                 // every sequence has one token: the thread that forms a channel's sum moves the slot on
 };
+
+// The sum over the taps of channel c for the token at place i of its step, whose inputs lie at first ..; with
+// a.shift (i is 0) the slot moves on by one, read and rewritten by the one thread that has the channel.
+__device__ __forceinline__ float conv_channel(const ShortConv& a, int first, int i, bool fresh, float* past, int c) {
+  const int back = a.taps - 1;
+  float acc = a.bias != nullptr ? a.bias[c] : 0.f;
+  for (int j = 0; j < a.taps; ++j) {
+    const int idx = i - back + j;                       // place in the step of the tap's input
+    float x;
+    if (idx >= 0) x = a.buf[(size_t)(first + idx) * a.stride + a.col + c];
+    else x = fresh ? 0.f : past[(size_t)(back + idx) * a.C + c];
+    if (a.shift && j > 0) past[(size_t)(j - 1) * a.C + c] = x;
+    acc += a.w[(size_t)c * a.taps + j] * x;
+  }
+  return acc;
+}
 
 // One wavefront per (token, head of the unit part | 256 other channels).
 __global__ __launch_bounds__(64) void short_conv_kernel(const ShortConv a) {
@@ -122,8 +210,7 @@ __global__ __launch_bounds__(64) void short_conv_kernel(const ShortConv a) {
   const int first = a.cu_q[s];
   const int i = t - first;                                  // place of the token in its step
   const bool fresh = a.positions[first] == 0;               // the sequence starts in this step
-  const float* past = a.state + (size_t)a.slots[s] * a.state_stride + a.state_off;
-  const int back = a.taps - 1;
+  float* past = a.state + (size_t)a.slots[s] * a.state_stride + a.state_off;
   float ss = 0.f;
   float y[4];
 #pragma unroll
@@ -131,14 +218,7 @@ __global__ __launch_bounds__(64) void short_conv_kernel(const ShortConv a) {
     const int c = c0 + lane + u * 64;
     y[u] = 0.f;
     if (lane + u * 64 < n) {
-      float acc = a.bias != nullptr ? a.bias[c] : 0.f;
-      for (int j = 0; j < a.taps; ++j) {
-        const int idx = i - back + j;                       // place in the step of the tap's input
-        float x;
-        if (idx >= 0) x = a.buf[(size_t)(first + idx) * a.stride + a.col + c];
-        else x = fresh ? 0.f : past[(size_t)(back + idx) * a.C + c];
-        acc += a.w[(size_t)c * a.taps + j] * x;
-      }
+      const float acc = conv_channel(a, first, i, fresh, past, c);
       y[u] = a.silu ? acc * sigmoidf_(acc) : acc;
       ss += y[u] * y[u];
     }
@@ -151,7 +231,11 @@ __global__ __launch_bounds__(64) void short_conv_kernel(const ShortConv a) {
   }
 #pragma unroll
   for (int u = 0; u < 4; ++u)
-    if (lane + u * 64 < n) a.out[(size_t)t * a.C + c0 + lane + u * 64] = y[u] * f;
+    if (lane + u * 64 < n) {
+      const size_t at = (size_t)t * a.C + c0 + lane + u * 64;
+      a.out[at] = y[u] * f;
+      if (a.rows != nullptr) a.rows[at] = from_f<act_t>(y[u] * f);
+    }
 }
 
 // The slot's new last inputs, after the kernel above has read the old ones: a thread per
@@ -178,7 +262,7 @@ extern "C" const char* sl_short_conv(const float* buf, int stride, int col, int 
                                      const float* bias, float* state, long long state_stride, int state_off, const int* cu_q,
                                      const int* positions, const int* tok_seq, const int* slots, int S, int T,
                                      int write, int unit_heads, int unit_dim, float unit_eps, int scaled_heads,
-                                     float scale, int silu, float* out, hipStream_t stream) {
+                                     float scale, int silu, float* out, void* rows, hipStream_t stream) {
   SL_CHECK(T >= 0 && S >= 0 && C > 0 && taps >= 1 && taps <= 64, "short_conv: sizes must be positive, taps <= 64");
   SL_CHECK(col >= 0 && col + C <= stride, "short_conv: the channels do not fit the rows");
   SL_CHECK(unit_heads >= 0 && (unit_heads == 0 || (unit_dim >= 1 && unit_dim <= 256)) &&
@@ -187,11 +271,12 @@ extern "C" const char* sl_short_conv(const float* buf, int stride, int col, int 
   SL_CHECK(state_off >= 0 && state_off + (long long)(taps - 1) * C <= state_stride,
            "short_conv: the last inputs do not fit the state slot");
   if (T == 0) return nullptr;
+  const int shift = write && taps > 1 && S == T;            // (no sequence is empty: one token each)
   const ShortConv a{buf, stride, col, C, taps, w, bias, state, state_stride, state_off, cu_q, positions, tok_seq,
-                    slots, unit_heads, unit_dim, scaled_heads, unit_eps, scale, silu, out};
+                    slots, unit_heads, unit_dim, scaled_heads, unit_eps, scale, silu, out, (act_t*)rows, shift};
   const int rest = C - unit_heads * unit_dim;
   short_conv_kernel<<<dim3(T, unit_heads + (rest + 255) / 256), 64, 0, stream>>>(a);
-  if (write && taps > 1) short_conv_state_kernel<<<dim3(S, (C + 255) / 256), 256, 0, stream>>>(a, S);
+  if (write && taps > 1 && !shift) short_conv_state_kernel<<<dim3(S, (C + 255) / 256), 256, 0, stream>>>(a, S);
   return sl_launch_status();
 }
 
@@ -306,7 +391,7 @@ extern "C" const char* sl_stream_conv(float* resid, int C, int taps, const float
   SL_CHECK(y == nullptr || (single && wy != nullptr), "stream_conv: a normed output is added for one token a sequence");
   if (T == 0) return nullptr;
   const ShortConv a{resid, C, 0, C, taps, w, nullptr, state, state_stride, state_off, cu_q, positions, tok_seq,
-                    slots, 0, 0, 0, 0.f, 1.f, 0, nullptr};
+                    slots, 0, 0, 0, 0.f, 1.f, 0, nullptr, nullptr, 0};
   if (single) {
     stream_step_kernel<<<T, C >= 2048 ? 1024 : (C >= 512 ? 512 : 256), 0, stream>>>(a, resid, (const act_t*)y, wy, eps,
                                                                                  write, (act_t*)out);
@@ -328,10 +413,11 @@ struct MatrixScan {
   float q_scale;
   const float* gates;        // delta: beta before its sigmoid at gates + t * gate_stride + beta_col + h;
   int gate_stride, i_col, f_col;   // matrix LSTM: the two gates before cap and squashing at i_col + h, f_col + h;
-                             // state-space: the step size before its bias and softplus at i_col + h
+                             // state-space: the step size before its bias and softplus at i_col + h;
+                             // delta with a decay per head: also the step size at f_col + h
   const float* rates;        // state-space, per head: dt = softplus(raw + step_bias[h]), the state keeps
   const float* step_bias;    // exp(-exp(rates[h]) dt) of itself and takes dt k v^T; the read-out adds
-  const float* skip;         // skip[h] v
+  const float* skip;         // skip[h] v.  (Delta with a decay per head: the same decay.)
   const float* lower;        // forget form: [H][D] lower bounds l of the gate; z lies where k lies else
   float cap;
   float* state;              // slot s at state + s * state_stride: S [H][Dv][D]; matrix LSTM: then n [H][D], m [H]
@@ -343,7 +429,7 @@ struct MatrixScan {
   float* out;                // [T][H][Dv]
 };
 
-enum { SCAN_DECAY = 0, SCAN_DELTA = 1, SCAN_LSTM = 2, SCAN_SSD = 3, SCAN_FORGET = 4 };
+enum { SCAN_DECAY = 0, SCAN_DELTA = 1, SCAN_LSTM = 2, SCAN_SSD = 3, SCAN_FORGET = 4, SCAN_DELTA_HEAD = 5 };
 constexpr int SCAN_ROWS = 8;      // key channels a lane owns: channels 8 p .. 8 p + 7
 
 // Sum over the P lanes that share a column (P a power of two, the lanes adjacent and aligned); every
@@ -388,7 +474,7 @@ __global__ __launch_bounds__(512) void matrix_scan_kernel(const MatrixScan a, in
   // The matrix LSTM's normaliser n is one more column of S whose value channel is always 1: the last
   // column group of every block carries it (every block the same one) and leaves max(|n . q|, e^-m) +
   // 1e-6 where the others leave their read-outs; these are divided by it when they leave LDS.
-  constexpr bool SCALAR = MODE == SCAN_LSTM || MODE == SCAN_SSD;      // one decay a head: no decays per channel in LDS
+  constexpr bool SCALAR = MODE == SCAN_LSTM || MODE == SCAN_SSD || MODE == SCAN_DELTA_HEAD;      // one decay a head: no decays per channel in LDS
   const int vcols = MODE == SCAN_LSTM ? cols - 1 : cols;
   const int half = CH * ((SCALAR ? 2 : 3) * Dp + 2 * cols + 4);
   const int oq = 0, ok = CH * Dp, oa = 2 * CH * Dp;          // [CH][Dp] each (no decays for the matrix LSTM)
@@ -444,7 +530,7 @@ __global__ __launch_bounds__(512) void matrix_scan_kernel(const MatrixScan a, in
       if (MODE != SCAN_DECAY && MODE != SCAN_FORGET && tid < 64 && tid < nt) {
         const float* gr = a.gates + (size_t)(t0 + tid) * a.gate_stride;
         g0 = gr[a.i_col + h];
-        if (MODE == SCAN_LSTM) g1 = gr[a.f_col + h];
+        if (MODE == SCAN_LSTM || MODE == SCAN_DELTA_HEAD) g1 = gr[a.f_col + h];
       }
     };
     // the read-outs of chunk c - 2 lie in the half that round c fills: they leave for memory first
@@ -492,6 +578,10 @@ __global__ __launch_bounds__(512) void matrix_scan_kernel(const MatrixScan a, in
           if (idx < nt * cols) base[ov + idx] = pv[e];
         }
         if (MODE == SCAN_DELTA && tid < nt) base[og + tid * 4] = sigmoidf_(g0);
+        if (MODE == SCAN_DELTA_HEAD && tid < nt) {
+          base[og + tid * 4] = expf(-expf(a.rates[h]) * softplusf_(g1 + a.step_bias[h]));
+          base[og + tid * 4 + 1] = sigmoidf_(g0);
+        }
         if (MODE == SCAN_SSD && tid < nt) {
           const float dt = softplusf_(g0 + a.step_bias[h]);
           base[og + tid * 4] = expf(-expf(a.rates[h]) * dt);
@@ -603,6 +693,17 @@ __global__ __launch_bounds__(512) void matrix_scan_kernel(const MatrixScan a, in
           S[i] = d[i] * S[i] + k[i] * u;
           part[i] = S[i] * q[i];
         }
+      } else if (MODE == SCAN_DELTA_HEAD) {
+        // (g S)^T k = g (S^T k): one factor for the whole column
+#pragma unroll
+        for (int i = 0; i < ROWS; ++i) part[i] = S[i] * k[i];
+        const float keep = sg[tt * 4];
+        const float u = sg[tt * 4 + 1] * (v - keep * group_sum(rows_sum<ROWS>(part), P));
+#pragma unroll
+        for (int i = 0; i < ROWS; ++i) {
+          S[i] = keep * S[i] + k[i] * u;
+          part[i] = S[i] * q[i];
+        }
       } else {
         const float keep = sg[tt * 4], av = sg[tt * 4 + 1] * v;     // (v is 1 in the column that carries n)
 #pragma unroll
@@ -643,12 +744,12 @@ extern "C" const char* sl_matrix_scan(int mode, const float* src, int src_stride
                                       const float* rates, const float* step_bias, const float* skip, const float* lower, float* state, long long state_stride,
                                       const int* cu_q, const int* positions,
                                       const int* slots, int S, int T, int write, float* out, hipStream_t stream) {
-  SL_CHECK(mode >= 0 && mode <= 4, "matrix_scan: unknown mode");
+  SL_CHECK(mode >= 0 && mode <= 5, "matrix_scan: unknown mode");
   SL_CHECK(S >= 0 && T >= 0 && H > 0 && G > 0 && H % G == 0 && Dv > 0, "matrix_scan: sizes must be positive");
   SL_CHECK(D >= 1 && D <= 64 * SCAN_ROWS, "matrix_scan: at most 512 key channels a head");
   SL_CHECK(q_col >= 0 && k_col >= 0 && v_col >= 0 && q_col + G * D <= src_stride && k_col + G * D <= src_stride &&
            v_col + H * Dv <= src_stride, "matrix_scan: q, k or v do not fit the rows");
-  SL_CHECK(mode == SCAN_LSTM || mode == SCAN_SSD || mode == SCAN_FORGET || log_decay != nullptr, "matrix_scan: decays are missing");
+  SL_CHECK(mode == SCAN_LSTM || mode == SCAN_SSD || mode == SCAN_FORGET || mode == SCAN_DELTA_HEAD || log_decay != nullptr, "matrix_scan: decays are missing");
   SL_CHECK(mode != SCAN_FORGET || (lower != nullptr && G == H), "matrix_scan: the forget form needs a bound per channel, and its gates per head");
   SL_CHECK(mode != SCAN_SSD || (rates != nullptr && step_bias != nullptr && skip != nullptr),
            "matrix_scan: the state-space form needs rates, step biases and skips per head");
@@ -656,6 +757,8 @@ extern "C" const char* sl_matrix_scan(int mode, const float* src, int src_stride
            "matrix_scan: gates are missing or do not fit their rows");
   SL_CHECK(mode != SCAN_LSTM || (f_col >= 0 && f_col + H <= gate_stride && cap > 0.f),
            "matrix_scan: the forget gates do not fit their rows");
+  SL_CHECK(mode != SCAN_DELTA_HEAD || (f_col >= 0 && f_col + H <= gate_stride && rates != nullptr && step_bias != nullptr),
+           "matrix_scan: a decay per head needs its step sizes within the rows, rates and step biases");
   const long long need = (long long)H * Dv * D + (mode == SCAN_LSTM ? (long long)H * D + H : 0);
   SL_CHECK(need <= state_stride, "matrix_scan: the state does not fit its slot");
   if (S == 0 || T == 0) return nullptr;
@@ -666,7 +769,7 @@ extern "C" const char* sl_matrix_scan(int mode, const float* src, int src_stride
   while (P * SCAN_ROWS < D) P <<= 1;
   const int cols = 256 / P, Dp = P * SCAN_ROWS;
   const int CH = min(min(16, 2048 / Dp), 8 * P);       // 8 values a thread of each kind a chunk
-  const bool scalar = mode == SCAN_LSTM || mode == SCAN_SSD;
+  const bool scalar = mode == SCAN_LSTM || mode == SCAN_SSD || mode == SCAN_DELTA_HEAD;
   const size_t lds = 2 * (size_t)CH * ((scalar ? 2 : 3) * Dp + 2 * cols + 4) * sizeof(float);   // two halves
   const MatrixScan a{src, src_stride, q_col, k_col, v_col, H, G, D, Dv, log_decay, q_scale, gates, gate_stride,
                      i_col, f_col, rates, step_bias, skip, lower, cap, state, state_stride, cu_q, positions, slots, write, out};
@@ -675,6 +778,7 @@ extern "C" const char* sl_matrix_scan(int mode, const float* src, int src_stride
   if (mode == SCAN_DECAY) matrix_scan_kernel<SCAN_DECAY, SCAN_ROWS><<<grid, 512, lds, stream>>>(a, P, CH);
   else if (mode == SCAN_DELTA) matrix_scan_kernel<SCAN_DELTA, SCAN_ROWS><<<grid, 512, lds, stream>>>(a, P, CH);
   else if (mode == SCAN_SSD) matrix_scan_kernel<SCAN_SSD, SCAN_ROWS><<<grid, 512, lds, stream>>>(a, P, CH);
+  else if (mode == SCAN_DELTA_HEAD) matrix_scan_kernel<SCAN_DELTA_HEAD, SCAN_ROWS><<<grid, 512, lds, stream>>>(a, P, CH);
   else if (mode == SCAN_FORGET) matrix_scan_kernel<SCAN_FORGET, SCAN_ROWS><<<grid, 512, lds, stream>>>(a, P, CH);
   else matrix_scan_kernel<SCAN_LSTM, SCAN_ROWS><<<grid, 512, lds, stream>>>(a, P, CH);
   return sl_launch_status();
@@ -737,7 +841,8 @@ extern "C" const char* sl_head_norm_gate(const float* o, int T, int H, int Dv, c
 // With taps given, the row's first conv_C channels first pass a short causal convolution over time
 // (no bias, no activation; the sums of short_conv_kernel in the same order): the block leaves its
 // token's sums in LDS and goes on from there, so the convolved rows never reach memory.  The
-// state's new last inputs are written by short_conv_state_kernel, launched behind this one.
+// state's new last inputs are written here when every sequence has one token (a channel is one thread's),
+// else by short_conv_state_kernel, launched behind this one.  G 0: the row holds queries only.
 __global__ void projnorm_rope_store_kernel(const float* __restrict__ buf, int stride, int H, int G, int D, int Dv,
                                            const float* __restrict__ qw, const float* __restrict__ kw, float eps,
                                            int rot, const float* __restrict__ cosv, const float* __restrict__ sinv,
@@ -753,19 +858,8 @@ __global__ void projnorm_rope_store_kernel(const float* __restrict__ buf, int st
     const int first = cv.cu_q[s];
     const int i = (int)t - first;
     const bool fresh = cv.positions[first] == 0;
-    const float* past = cv.state + (size_t)cv.slots[s] * cv.state_stride + cv.state_off;
-    const int back = cv.taps - 1;
-    for (int c = threadIdx.x; c < cv.C; c += blockDim.x) {
-      float acc = 0.f;
-      for (int j = 0; j < cv.taps; ++j) {
-        const int idx = i - back + j;
-        float x;
-        if (idx >= 0) x = buf[(size_t)(first + idx) * stride + c];
-        else x = fresh ? 0.f : past[(size_t)(back + idx) * cv.C + c];
-        acc += cv.w[(size_t)c * cv.taps + j] * x;
-      }
-      convolved[c] = acc;
-    }
+    float* past = cv.state + (size_t)cv.slots[s] * cv.state_stride + cv.state_off;
+    for (int c = threadIdx.x; c < cv.C; c += blockDim.x) convolved[c] = conv_channel(cv, first, i, fresh, past, c);
     __syncthreads();
     row = convolved;
   }
@@ -777,7 +871,7 @@ __global__ void projnorm_rope_store_kernel(const float* __restrict__ buf, int st
     for (int e = threadIdx.x; e < nq; e += blockDim.x) sq += row[e] * row[e];
     for (int e = threadIdx.x; e < nk; e += blockDim.x) sk += row[nq + e] * row[nq + e];
     iq = 1.f / sqrtf(block_sum(sq, scratch) / (float)nq + eps);
-    ik = 1.f / sqrtf(block_sum(sk, scratch) / (float)nk + eps);
+    if (nk > 0) ik = 1.f / sqrtf(block_sum(sk, scratch) / (float)nk + eps);
   }
   const int half = rot / 2;
   const float* cs = cosv != nullptr ? cosv + t * half : nullptr;
@@ -891,12 +985,13 @@ extern "C" const char* sl_projnorm_rope_store(const float* buf, int stride, int 
                                               long long state_stride, int state_off, const int* cu_q,
                                               const int* positions, const int* tok_seq, const int* state_slots,
                                               int S, int write_state, hipStream_t stream) {
-  SL_CHECK(T >= 0 && H > 0 && G > 0 && D > 0 && Dv > 0 && page > 0, "projnorm_rope_store: sizes must be positive");
+  SL_CHECK(T >= 0 && H > 0 && G >= 0 && D > 0 && Dv > 0 && page > 0, "projnorm_rope_store: sizes must be positive");
+  SL_CHECK(G > 0 || slots == nullptr, "projnorm_rope_store: there are no keys to store");
   SL_CHECK((long long)(H + G) * D <= stride && v_col >= 0 && v_col + (long long)G * Dv <= stride,
            "projnorm_rope_store: q, k and v do not fit the rows");
   SL_CHECK(rot >= 0 && rot % 2 == 0 && rot <= D, "projnorm_rope_store: the rotated width must be even and within a head");
   SL_CHECK(rot == 0 || (cosv != nullptr && sinv != nullptr), "projnorm_rope_store: cos and sin are missing");
-  SL_CHECK((qw == nullptr) == (kw == nullptr), "projnorm_rope_store: both gains or neither");
+  SL_CHECK((qw == nullptr) == (kw == nullptr) || G == 0, "projnorm_rope_store: both gains or neither");
   SL_CHECK(slots == nullptr || (kc != nullptr && vc != nullptr), "projnorm_rope_store: pages are missing");
   ShortConv cv{};
   size_t lds = 0;
@@ -909,7 +1004,7 @@ extern "C" const char* sl_projnorm_rope_store(const float* buf, int stride, int 
     SL_CHECK(state_off >= 0 && state_off + (long long)(taps - 1) * conv_C <= state_stride,
              "projnorm_rope_store: the last inputs do not fit the state slot");
     cv = ShortConv{buf, stride, 0, conv_C, taps, taps_w, nullptr, state, state_stride, state_off, cu_q, positions,
-                   tok_seq, state_slots, 0, 0, 0, 0.f, 1.f, 0, nullptr};
+                   tok_seq, state_slots, 0, 0, 0, 0.f, 1.f, 0, nullptr, nullptr, 0};
     lds = (size_t)conv_C * sizeof(float);
   }
   if (T == 0) return nullptr;
@@ -921,10 +1016,12 @@ extern "C" const char* sl_projnorm_rope_store(const float* buf, int stride, int 
   if ((qw != nullptr && per_head) || (qw == nullptr && H + 2 * G <= 65535 && T < 512))
     rope_store_heads_kernel<<<dim3(T, H + 2 * G), 64, 0, stream>>>(buf, stride, H, G, D, Dv, qw, kw, eps, rot, cosv, sinv, slots,
                                                                    (act_t*)kc, (act_t*)vc, page, (act_t*)q_out, v_col, cv);
-  else   // (a step of few tokens has few blocks: wider ones shorten each block's loops over the row)
+  else {   // (a step of few tokens has few blocks: wider ones shorten each block's loops over the row)
+    cv.shift = taps_w != nullptr && write_state && taps > 1 && S == T;
     projnorm_rope_store_kernel<<<T, T <= 64 ? 1024 : 256, lds, stream>>>(buf, stride, H, G, D, Dv, qw, kw, eps, rot, cosv, sinv, slots,
                                                         (act_t*)kc, (act_t*)vc, page, (act_t*)q_out, v_col, cv);
-  if (taps_w != nullptr && write_state && taps > 1)
+  }
+  if (taps_w != nullptr && write_state && taps > 1 && !cv.shift)
     short_conv_state_kernel<<<dim3(S, (conv_C + 255) / 256), 256, 0, stream>>>(cv, S);
   return sl_launch_status();
 }

@@ -1,7 +1,9 @@
 // Routed experts: every token goes through the `top` experts with the largest router logits,
 // weighted by the softmax over those logits only; or (shares over all experts) with the largest
 // softmax shares plus a correction per expert, weighted by their shares, divided by their sum
-// and multiplied by a constant.  The last experts may be ones without matrices that hand their
+// and multiplied by a constant; or with the largest logits, weighted by their sigmoids, which
+// multiply an expert's input instead of its output (as a factor of its first products' sums:
+// W (s x) = s (W x)).  The last experts may be ones without matrices that hand their
 // input through.
 //
 //   route       per token the chosen experts and their shares (float), one wavefront a token
@@ -24,11 +26,12 @@
 // ------------------------------------------------------------------ route
 // One wavefront per token.  Largest first; among equal logits the lower index wins.
 // over_all: the numbers compared are softmax(z)[e] + correction[e] over all E, and a chosen
-// expert's share is softmax(z)[e] / (sum over the chosen + 1e-20) * scale.
+// expert's share is softmax(z)[e] / (sum over the chosen + 1e-20) * scale.  sigmoid: the logits are
+// compared, and a chosen expert's share is the sigmoid of its own.
 __global__ __launch_bounds__(64) void route_kernel(const float* __restrict__ logits, int stride, int E, int top,
                                                    int* __restrict__ chosen, float* __restrict__ shares,
                                                    int over_all, const float* __restrict__ correction,
-                                                   float scale) {
+                                                   float scale, int sigmoid) {
   const size_t t = blockIdx.x;
   const int lane = threadIdx.x;
   const float* z = logits + t * stride;
@@ -90,6 +93,13 @@ __global__ __launch_bounds__(64) void route_kernel(const float* __restrict__ log
     if (lane < top) {
       chosen[t * top + lane] = mine_e;
       shares[t * top + lane] = w / (sum + 1e-20f) * scale;
+    }
+    return;
+  }
+  if (sigmoid) {
+    if (lane < top) {
+      chosen[t * top + lane] = mine_e;
+      shares[t * top + lane] = 1.f / (1.f + expf(-mine));
     }
     return;
   }
@@ -156,7 +166,8 @@ __global__ __launch_bounds__(1024) void group_kernel(const int* __restrict__ cho
 extern "C" const char* sl_route_tokens(const float* logits, int stride, int T, int E, int top, int* chosen,
                                        float* shares, int* order, int* place_of, int* tiles, int max_tiles,
                                        int tile_rows, int over_all, const float* correction, float scale,
-                                       int E_real, hipStream_t stream) {
+                                       int E_real, int sigmoid, hipStream_t stream) {
+  SL_CHECK(!(over_all && sigmoid), "route_tokens: shares over all or sigmoids");
   SL_CHECK(T >= 0 && E >= 1 && E <= 4096 && top >= 1 && top <= 64 && top <= E && E <= stride,
            "route_tokens: at most 4096 experts within the rows, at most 64 choices");
   SL_CHECK(E_real >= 0 && E_real <= E && (over_all || correction == nullptr),
@@ -164,7 +175,7 @@ extern "C" const char* sl_route_tokens(const float* logits, int stride, int T, i
   SL_CHECK(tile_rows == 16 || tile_rows == 64 || tile_rows == 128, "route_tokens: row tiles hold 16, 64 or 128 rows");
   SL_CHECK(max_tiles >= ((long long)T * top + tile_rows - 1) / tile_rows + E, "route_tokens: too few tile entries");
   if (T == 0) return nullptr;
-  route_kernel<<<T, 64, 0, stream>>>(logits, stride, E, top, chosen, shares, over_all, correction, scale);
+  route_kernel<<<T, 64, 0, stream>>>(logits, stride, E, top, chosen, shares, over_all, correction, scale, sigmoid);
   group_kernel<<<1, 1024, 3 * E * sizeof(int), stream>>>(chosen, T * top, E, E_real, max_tiles, tile_rows, order,
                                                          place_of, tiles);
   return sl_launch_status();
@@ -185,6 +196,7 @@ struct Grouped {
   float* out_f32;            // plain: [rows][N]
   int act;                   // the activation (common.h); 0 with out_f32
   float limit;               // the clamped gate's bound
+  const float* row_scale;    // with order: the sums of row r are multiplied by row_scale[order[r]] first; or nullptr
   int max_tiles, col_blocks; // the matrix-core kernels' launch: max_tiles x col_blocks workgroups in a row
 };
 
@@ -248,11 +260,14 @@ __global__ __launch_bounds__(256) void grouped_product_kernel(const Grouped a) {
     }
   }
   if (r >= rows) return;
+  const float rs = a.row_scale != nullptr ? a.row_scale[a.order[row0 + r]] : 1.f;
 #pragma unroll
   for (int u = 0; u < 4; ++u) {
     const int n = n0 + l + 16 * u;
     if (n >= a.N) continue;
     const size_t at = (size_t)(row0 + r) * a.N + n;
+    acc[u] *= rs;
+    if (GATED) acc2[u] *= rs;
     if (GATED) a.out_act[at] = from_f<act_t>(sl_gated(acc[u], acc2[u], a.act, a.limit));
     else if (a.act) a.out_act[at] = from_f<act_t>(sl_act(acc[u], a.act));
     else a.out_f32[at] = acc[u];
@@ -331,6 +346,14 @@ __global__ __launch_bounds__(64 * WR * WC) void grouped_product_mfma_kernel(cons
   for (int v = 0; v < NT; ++v) {
     if (16 * v + i >= rows) continue;
     const size_t at = (size_t)(row0 + 16 * v + i) * a.N + n0 + 4 * gq;
+    if (a.row_scale != nullptr) {
+      const float rs = a.row_scale[a.order[row0 + 16 * v + i]];
+#pragma unroll
+      for (int u = 0; u < NU; ++u) {
+        acc[v][u] *= rs;
+        if (GATED) acc2[v][u] *= rs;
+      }
+    }
 #pragma unroll
     for (int u = 0; u < NU; ++u) {
       if (n0 + 16 * u >= a.N) continue;
@@ -447,6 +470,13 @@ __global__ __launch_bounds__(256, 2) void grouped_product_staged_kernel(const Gr
   for (int v = 0; v < NT; ++v) {
     if (16 * v + i >= rows) continue;
     const size_t at = (size_t)(row0 + 16 * v + i) * a.N + n0 + 4 * gq;
+    if (a.row_scale != nullptr) {
+      const float rs = a.row_scale[a.order[row0 + 16 * v + i]];
+#pragma unroll
+      for (int u = 0; u < NU * MATS; ++u) {
+        acc[v][u] *= rs;
+      }
+    }
 #pragma unroll
     for (int u = 0; u < NU; ++u) {
       if (n0 + 16 * u >= a.N) continue;
@@ -470,16 +500,17 @@ __global__ __launch_bounds__(256, 2) void grouped_product_staged_kernel(const Gr
 
 extern "C" const char* sl_grouped_product(const void* x, const int* order, int top, const void* w, const int* tiles,
                                           int w_tiled, int max_tiles, int tile_rows, int N, int K, int gated,
-                                          int act, float limit, void* out, hipStream_t stream) {
+                                          int act, float limit, const float* row_scale, void* out, hipStream_t stream) {
   // gated: act(gate) * up into the activation type; else act != 0: act(W x) into the activation type;
   // else plain float sums
   SL_CHECK(max_tiles >= 0 && N > 0 && K > 0 && top >= 1, "grouped_product: sizes must be positive");
   SL_CHECK(act >= 0 && act <= SL_ACT_CLAMPED_SWISH && (!gated || act) && (gated || act != SL_ACT_CLAMPED_SWISH),
            "grouped_product: unknown activation, a gate without one, or the clamped form without a gate");
+  SL_CHECK(row_scale == nullptr || order != nullptr, "grouped_product: factors per row go with the pairs' order");
   SL_CHECK(tile_rows == 16 || tile_rows == 64 || tile_rows == 128, "grouped_product: row tiles hold 16, 64 or 128 rows");
   if (max_tiles == 0) return nullptr;
   Grouped a{(const act_t*)x, order, top, (const act_t*)w, w_tiled, tiles, tile_rows / RT_ROWS, N, K,
-            act ? (act_t*)out : nullptr, act ? nullptr : (float*)out, act, limit, max_tiles, 1};
+            act ? (act_t*)out : nullptr, act ? nullptr : (float*)out, act, limit, row_scale, max_tiles, 1};
 #if !defined(SL_F32)
   if (K % 32 == 0 && N % 16 == 0 && (uintptr_t)x % 16 == 0 && (uintptr_t)w % 16 == 0 && (uintptr_t)out % 16 == 0) {
     // (a one-dimensional launch of max_tiles x col_blocks workgroups, rounded up to the eight dies)
@@ -512,7 +543,7 @@ extern "C" const char* sl_grouped_product(const void* x, const int* order, int t
 
 // ------------------------------------------------------------------ combine
 // out[t] = g[t] base[t] + sum_k shares[t][k] * y[place_of[t top + k]], float sums, choices in their order;
-// g[t] = sigmoid(base_gate[t * gate_stride]) when base_gate is given, else 1.  A choice from
+// g[t] = sigmoid(base_gate[t * gate_stride]) when base_gate is given, else 1 (shares == nullptr: all 1).  A choice from
 // E_real on (chosen given) is an expert that hands its input through: it adds share * x[t].
 __global__ __launch_bounds__(256) void routed_combine_kernel(const float* __restrict__ y,
                                                              const int* __restrict__ place_of,
@@ -528,7 +559,7 @@ __global__ __launch_bounds__(256) void routed_combine_kernel(const float* __rest
   if (threadIdx.x < top) {
     const bool through = chosen != nullptr && chosen[t * top + threadIdx.x] >= E_real;
     place[threadIdx.x] = through ? -1 : place_of[t * top + threadIdx.x];
-    share[threadIdx.x] = shares[t * top + threadIdx.x];
+    share[threadIdx.x] = shares != nullptr ? shares[t * top + threadIdx.x] : 1.f;
   }
   __syncthreads();
   const int c = blockIdx.y * 256 + threadIdx.x;

@@ -17,6 +17,7 @@ struct WindowAttention {
   float scale;
   float softcap;             // c > 0: the scaled score becomes c tanh(score / c); 0: left as it is
   int window;                // 0: every earlier key
+  int chunk;                 // > 0: keys of the query's own chunk of so many positions; 0: no chunks
   int keep_first;
   const float* slopes;       // [nh] or nullptr
   const float* sinks;        // [nh] or nullptr
@@ -29,6 +30,16 @@ struct WindowAttention {
   float* part_o;             // [tokens][nh][nsplit][Dv]
   float* part_ml;            // [tokens][nh][nsplit][2]
 };
+
+// The first key that a query at position pos sees by window and chunk (kept first keys aside).
+__device__ __forceinline__ int first_key(const WindowAttention& a, int pos) {
+  int lo = a.window > 0 && pos - a.window + 1 > 0 ? pos - a.window + 1 : 0;
+  if (a.chunk > 0) {
+    const int c = pos - pos % a.chunk;
+    lo = c > lo ? c : lo;
+  }
+  return lo;
+}
 
 __device__ __forceinline__ float sigmoidf_(float x) { return 1.f / (1.f + expf(-x)); }
 

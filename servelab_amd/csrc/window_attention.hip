@@ -5,6 +5,7 @@
 //     key rows (a cached latent that serves as key and as value);
 //   * a window that also keeps the first tokens: the query at position i of its
 //     sequence sees key j <= i when i - j < window or j < keep_first;
+//   * chunks: it sees only keys of its own chunk of positions (or j < keep_first);
 //   * capped scores: the scaled score s becomes c tanh(s / c);
 //   * a distance bias: slope_h * (i - j) is taken off the scaled score;
 //   * a sink: exp(sink_h) enters the softmax's denominator once, without a key
@@ -57,13 +58,12 @@ __global__ __launch_bounds__(WA_THREADS) void window_attention_kernel(const Wind
   const bool live = c < ncols;
   const int tok = live ? c / g : 0, head = kvh * g + (live ? c % g : 0);
   const int pos_c = live ? pos0 + tok : -1;
-  const int lo_c = a.window > 0 && pos_c - a.window + 1 > 0 ? pos_c - a.window + 1 : 0;
+  const int lo_c = live ? first_key(a, pos_c) : 0;
   const float slope = a.slopes != nullptr ? a.slopes[head] : 0.f;
   const int tok_first = c0 / g;
   const int c_last = c0 + WA_COLS - 1 < ncols - 1 ? c0 + WA_COLS - 1 : ncols - 1;
   const int kmax = pos0 + c_last / g;
-  int kmin = 0;
-  if (a.window > 0 && pos0 + tok_first - a.window + 1 > 0) kmin = pos0 + tok_first - a.window + 1;
+  const int kmin = first_key(a, pos0 + tok_first);
   const int keep = a.keep_first < kmin ? a.keep_first : kmin;      // keys [0, keep) and [kmin, kmax]
   // blocks [0, nA) hold the kept first keys, blocks [firstB, firstB + nB) the window
   const int nA = keep > 0 ? (keep - 1) / KB + 1 : 0;
@@ -219,7 +219,7 @@ static const char* launch_window_attention(const WindowAttention& a, dim3 grid, 
 extern "C" const char* sl_window_attention(
     const void* q, int q_stride, const void* kc, const void* vc, const int* tables, int max_pages,
     const int* cu_q, const int* positions, int num_seqs, int max_q_len, int num_tokens, int nh,
-    int nkv, int Dk, int Dv, int page, float scale, float softcap, int window, int keep_first, const float* slopes,
+    int nkv, int Dk, int Dv, int page, float scale, float softcap, int window, int chunk, int keep_first, const float* slopes,
     const float* sinks, const void* gate, int gate_stride, const float* channel_gate, int channel_stride, void* out,
     int nsplit, float* part_o, float* part_ml, hipStream_t stream) {
   SL_CHECK(num_seqs >= 0 && max_q_len >= 1 && nh > 0 && nkv > 0 && nh % nkv == 0,
@@ -228,7 +228,8 @@ extern "C" const char* sl_window_attention(
   SL_CHECK(vc != nullptr || Dv <= Dk, "window attention: values read from key rows cannot be wider than a key");
   SL_CHECK(page == 16 || page == 32 || page == 64, "window attention: page size must be 16, 32 or 64");
   SL_CHECK(nkv <= 65535 && num_seqs <= 65535, "window attention: grid too large");
-  SL_CHECK(window >= 0 && keep_first >= 0 && softcap >= 0.f, "window attention: window, keep_first and the cap must be >= 0");
+  SL_CHECK(window >= 0 && chunk >= 0 && keep_first >= 0 && softcap >= 0.f,
+           "window attention: window, chunk, keep_first and the cap must be >= 0");
   SL_CHECK(nsplit >= 1 && nsplit <= 64, "window attention: 1..64 shares of the keys");
   SL_CHECK(nsplit == 1 || (part_o != nullptr && part_ml != nullptr),
            "window attention: shares of the keys need the partial buffers");
@@ -239,7 +240,7 @@ extern "C" const char* sl_window_attention(
   const long long tiles = (cols + WA_COLS - 1) / WA_COLS;
   SL_CHECK(tiles * nsplit <= 1 << 30, "window attention: too many column tiles");
   const WindowAttention a{(const act_t*)q, q_stride, (const act_t*)kc, (const act_t*)vc, tables, max_pages,
-                          cu_q, positions, nh, nkv, Dk, Dv, page, scale, softcap, window, keep_first, slopes, sinks,
+                          cu_q, positions, nh, nkv, Dk, Dv, page, scale, softcap, window, chunk, keep_first, slopes, sinks,
                           (const act_t*)gate, gate_stride, channel_gate, channel_stride, (act_t*)out, nsplit, part_o,
                           part_ml};
   const dim3 grid((unsigned)(tiles * nsplit), nkv, num_seqs);

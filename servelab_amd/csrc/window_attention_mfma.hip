@@ -96,8 +96,7 @@ __global__ __launch_bounds__(THREADS) void window_attention_mfma_kernel(const Wi
   const int tok_first = c0 / g;
   const int c_last = c0 + COLS - 1 < ncols - 1 ? c0 + COLS - 1 : ncols - 1;
   const int kmax = pos0 + c_last / g;
-  int kmin = 0;
-  if (a.window > 0 && pos0 + tok_first - a.window + 1 > 0) kmin = pos0 + tok_first - a.window + 1;
+  const int kmin = first_key(a, pos0 + tok_first);
   const int keep = a.keep_first < kmin ? a.keep_first : kmin;
   const int nA = keep > 0 ? (keep - 1) / 32 + 1 : 0;
   int firstB = kmin / 32;
@@ -124,11 +123,11 @@ __global__ __launch_bounds__(THREADS) void window_attention_mfma_kernel(const Wi
   if (!live) c = ncols - 1;
   const int tok = c / g, head = kvh * g + c % g;
   const int pos_c = pos0 + tok;
-  const int lo_c = a.window > 0 && pos_c - a.window + 1 > 0 ? pos_c - a.window + 1 : 0;
+  const int lo_c = first_key(a, pos_c);
   // every column of the wavefront sees all of a block [kb, kb + 31] when kb + 31 <= pos_lo and (kb >= lo_hi
   // or the block lies within the kept first tokens)
   const int pos_lo = pos0 + (wave_live ? cw0 : 0) / g, pos_hi = pos0 + (wave_live ? cw1 : 0) / g;
-  const int lo_hi = a.window > 0 && pos_hi - a.window + 1 > 0 ? pos_hi - a.window + 1 : 0;
+  const int lo_hi = first_key(a, pos_hi);
   const float scale2 = a.scale * LOG2E;
   const bool capped = a.softcap > 0.f;
   const float cap2 = a.softcap * LOG2E, uncap = capped ? a.scale / a.softcap : 0.f;
@@ -393,7 +392,7 @@ extern "C" int sl_window_attention_mfma_lds_bytes() {
 extern "C" const char* sl_window_attention_mfma(
     const void* q, int q_stride, const void* kc, const void* vc, const int* tables, int max_pages,
     const int* cu_q, const int* positions, int num_seqs, int max_q_len, int num_tokens, int nh,
-    int nkv, int Dk, int Dv, int page, float scale, float softcap, int window, int keep_first, const float* slopes,
+    int nkv, int Dk, int Dv, int page, float scale, float softcap, int window, int chunk, int keep_first, const float* slopes,
     const float* sinks, const void* gate, int gate_stride, const float* channel_gate, int channel_stride, void* out,
     int nsplit, float* part_o, float* part_ml, hipStream_t stream) {
   SL_CHECK(Dk == DK && Dv == DV && (vc == nullptr) == VK, "window attention (matrix cores): built for other widths");
@@ -401,7 +400,8 @@ extern "C" const char* sl_window_attention_mfma(
            "window attention: heads must be a positive multiple of kv heads");
   SL_CHECK(page == 16 || page == 32 || page == 64, "window attention: page size must be 16, 32 or 64");
   SL_CHECK(nkv <= 65535 && num_seqs <= 65535, "window attention: grid too large");
-  SL_CHECK(window >= 0 && keep_first >= 0 && softcap >= 0.f, "window attention: window, keep_first and the cap must be >= 0");
+  SL_CHECK(window >= 0 && chunk >= 0 && keep_first >= 0 && softcap >= 0.f,
+           "window attention: window, chunk, keep_first and the cap must be >= 0");
   SL_CHECK(nsplit >= 1 && nsplit <= 64, "window attention: 1..64 shares of the keys");
   SL_CHECK(nsplit == 1 || (part_o != nullptr && part_ml != nullptr),
            "window attention: shares of the keys need the partial buffers");
@@ -412,7 +412,7 @@ extern "C" const char* sl_window_attention_mfma(
            "window attention (matrix cores): operands must be 16-byte aligned");
   if (num_seqs == 0 || num_tokens == 0) return nullptr;
   const WindowAttention a{(const act_t*)q, q_stride, (const act_t*)kc, (const act_t*)vc, tables, max_pages,
-                          cu_q, positions, nh, nkv, Dk, Dv, page, scale, softcap, window, keep_first, slopes, sinks,
+                          cu_q, positions, nh, nkv, Dk, Dv, page, scale, softcap, window, chunk, keep_first, slopes, sinks,
                           (const act_t*)gate, gate_stride, channel_gate, channel_stride, (act_t*)out, nsplit, part_o,
                           part_ml};
   const long long cols = (long long)max_q_len * (nh / nkv);

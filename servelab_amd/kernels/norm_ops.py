@@ -10,20 +10,21 @@ from .values import (Deferred, KernelError, PartialSums, ScaledRows, TiledRows, 
 
 class NormOps:
     # ------------------------------------------------------------ embedding
-    def embed(self, ids, table, scale=1.0, positions=None, pos_table=None):
+    def embed(self, ids, table, scale=1.0, positions=None, pos_table=None, copies=0):
         """The rows of ``table`` at ``ids`` times ``scale``, as the float32 stream [T, H]; with
-        ``pos_table`` [P, H] the rows at ``positions`` (int32, each below P) are added, unscaled."""
+        ``pos_table`` [P, H] the rows at ``positions`` (int32, each below P) are added, unscaled.
+        ``copies`` s: the stream as s equal copies [T, s, H]."""
         T = ids.shape[0]
         V, H = table.shape
         self._check(ids, torch.int32, (T,), "ids")
         self._check(table, self.act_dtype, None, "embedding table")
-        out = self._new((T, H), torch.float32)
+        out = self._new((T, copies, H) if copies else (T, H), torch.float32)
         if pos_table is not None:
             self._check(positions, torch.int32, (T,), "positions")
             self._check(pos_table, self.act_dtype, (pos_table.shape[0], H), "position table")
         self._call("elementwise", "sl_embed", _p(ids), _p(table), _p(out), T, H, V, _c_float(scale),
                    _p(positions) if pos_table is not None else None, _p(pos_table),
-                   pos_table.shape[0] if pos_table is not None else 0)
+                   pos_table.shape[0] if pos_table is not None else 0, max(1, int(copies)))
         return out
 
     def stream_pair(self, resid, delta, other):
@@ -160,6 +161,45 @@ class NormOps:
         self._call("elementwise", "sl_activate", _p(x), _p(x), ctypes.c_longlong(x.numel()),
                    activation_code(activation, ("silu", "relu", "relu2", "gelu_tanh")))
         return x
+
+    MAX_STREAMS = 16              # copies of the stream that the kernel takes
+
+    def streams_norm(self, resid, outputs, mix, out, read, weight, bias, eps, center=True, rows=None):
+        """The norm a sublayer puts before itself over a stream kept in copies, ``resid`` [T, s, H] float32.
+        ``outputs``: up to two (y [T, H], gain or None, eps): the last sublayer's output is their sum, each
+        first RMS-normed where it has a gain; every copy becomes x_t <- sum_s mix[s, t] x_s + out[t] y, in
+        place (no ``outputs``: the copies stay as they are).  Then u = sum_s read[s] x_s (``read`` None: the
+        plain sum) and its layer norm (``center`` False: RMS norm) with gain ``weight`` and ``bias`` (or
+        None), as rows in the activation dtype.  ``rows`` (int32): only those rows are computed and
+        returned, and the copies stay as they are."""
+        self._check(resid, torch.float32, None, "residual stream")
+        if resid.dim() != 3 or not 1 <= resid.shape[1] <= self.MAX_STREAMS:
+            raise KernelError(f"the stream must be [T, copies, H] with at most {self.MAX_STREAMS} copies")
+        T, S, H = resid.shape
+        self._check(weight, torch.float32, (H,), "norm weight")
+        if bias is not None:
+            self._check(bias, torch.float32, (H,), "norm bias")
+        if len(outputs) > 2:
+            raise KernelError("streams_norm: at most two outputs join the stream at a time")
+        for y, gain, _ in outputs:
+            self._check(y, self.act_dtype, (T, H), "sublayer output")
+            if gain is not None:
+                self._check(gain, torch.float32, (H,), "output norm weight")
+        if outputs:
+            self._check(mix, torch.float32, (S, S), "mix")
+            self._check(out, torch.float32, (S,), "out")
+        if read is not None:
+            self._check(read, torch.float32, (S,), "read")
+        if rows is not None:
+            self._check(rows, torch.int32, (rows.shape[0],), "rows")
+        R = T if rows is None else rows.shape[0]
+        result = self._new((R, H))
+        y1, g1, e1 = outputs[0] if outputs else (None, None, 0.0)
+        y2, g2, e2 = outputs[1] if len(outputs) > 1 else (None, None, 0.0)
+        self._call("norm", "sl_streams_norm", _p(resid), S, _p(y1), _p(g1), _c_float(e1), _p(y2), _p(g2), _c_float(e2),
+                   _p(mix) if outputs else None, _p(out) if outputs else None, _p(read), _p(rows), _p(weight), _p(bias),
+                   _c_float(eps), int(bool(center)), _p(result), R, H)
+        return result
 
     def add_normed_rmsnorm(self, resid, y, y_weight, y_eps, weight, eps, rows=None):
         """A sublayer's output ``y`` joins the float32 stream through an RMS norm of its own, and the

@@ -1,6 +1,6 @@
 """Calls for mixers that keep a matrix per head in a state slot, for a softmax attention whose q
 and k are normed over the whole projection, for an RMS norm on a sublayer's output, and for
-routed experts.  Their libraries (``recurrent``, ``routed``) are compiled when a model first
+routed experts.  Their libraries (``recurrent``, ``selective``, ``routed``) are compiled when a model first
 asks for them.
 
 What is float32 here in both activation types: the input projections' sums as these calls read
@@ -15,8 +15,8 @@ from .values import KernelError, _c_float, _p, activation_code
 
 _ll = ctypes.c_longlong
 
-_EXPAND_MODES = {"plain": 0, "log_sigmoid": 1, "rate_softplus": 2}
-_SCAN_DECAY, _SCAN_DELTA, _SCAN_LSTM, _SCAN_SSD, _SCAN_FORGET = 0, 1, 2, 3, 4
+_EXPAND_MODES = {"plain": 0, "log_sigmoid": 1, "rate_softplus": 2, "softplus": 3}
+_SCAN_DECAY, _SCAN_DELTA, _SCAN_LSTM, _SCAN_SSD, _SCAN_FORGET, _SCAN_DELTA_HEAD = 0, 1, 2, 3, 4, 5
 _TILE_ROWS = (16, 64, 128)    # rows of a row tile of the grouped products (routed.hip)
 
 
@@ -44,6 +44,7 @@ class ExpertMatrices:
 
 
 class RecurrentOps:
+    SELECTIVE_SEGMENT = 64        # tokens of a segment of the selective scan
     ROUTED_WIDE_TILE_ROWS = 48    # rows an expert has on average from which row tiles hold 64 rows
 
     # ------------------------------------------------- norm on an output
@@ -96,7 +97,8 @@ class RecurrentOps:
 
     def lowrank_expand(self, buf, col, w2, bias, mode, heads=1, divisor=1.0, rates=None):
         """z = buf[:, col:col + rank] w2^T + bias as float32 [T, C]: "plain" z, "log_sigmoid"
-        logsigmoid(z) / divisor, "rate_softplus" -exp(rates[h]) softplus(z) with h = c // (C / heads)."""
+        logsigmoid(z) / divisor, "softplus" softplus(z), "rate_softplus" -exp(rates[h]) softplus(z) with
+        h = c // (C / heads)."""
         T, stride = self._f32_rows(buf, "projected rows")
         C, rank = w2.shape
         self._check(w2, torch.float32, None, "expansion matrix")
@@ -112,13 +114,14 @@ class RecurrentOps:
         return out
 
     def short_conv(self, buf, col, taps, state, state_off, batch, write, unit_heads=0, unit_dim=0,
-                   unit_eps=1e-6, scaled_heads=0, scale=1.0, bias=None, activation="silu"):
+                   unit_eps=1e-6, scaled_heads=0, scale=1.0, bias=None, activation="silu", want_rows=False):
         """silu (``activation`` None: nothing) of a causal convolution over time per channel of buf[:, col:col + C] (``taps``
         [C, n], the last one the token's own; ``bias`` [C] is added before the silu).  The n - 1 inputs before a step come from the
         sequence's state slot at ``state_off`` ([n - 1, C], zeros at a sequence's start), and the
         step's last n - 1 inputs go back there.  The first ``unit_heads`` heads of ``unit_dim``
         channels are divided by sqrt(sum x^2 + unit_eps), the first ``scaled_heads`` of them also
-        multiplied by ``scale``.  Returns float32 [T, C]."""
+        multiplied by ``scale``.  Returns float32 [T, C]; with ``want_rows`` the pair of it and the same
+        rows in the activation dtype."""
         T, stride = self._f32_rows(buf, "projected rows")
         C, n = taps.shape
         self._check(taps, torch.float32, None, "taps")
@@ -129,11 +132,12 @@ class RecurrentOps:
         self._sequences(batch, T)
         slot_size = self._state(state, state_off + (n - 1) * C)
         out = self._new((T, C), torch.float32)
+        rows = self._new((T, C)) if want_rows else None
         self._call(self._lazy("recurrent"), "sl_short_conv", _p(buf), stride, col, C, n, _p(taps), _p(bias), _p(state),
                    _ll(slot_size), state_off, _p(batch.cu_q), _p(batch.positions), _p(batch.tok_seq),
                    _p(batch.state_slots), batch.num_seqs, T, int(bool(write)), unit_heads, unit_dim,
-                   _c_float(unit_eps), scaled_heads, _c_float(scale), int(activation == "silu"), _p(out))
-        return out
+                   _c_float(unit_eps), scaled_heads, _c_float(scale), int(activation == "silu"), _p(out), _p(rows))
+        return (out, rows) if want_rows else out
 
     def stream_conv(self, resid, taps, state, state_off, batch, write, y=None, y_weight=None, y_eps=1e-6):
         """Rows x_t + sum_j taps[j] x_(t - n + 1 + j) of the float32 stream x, per channel, in the
@@ -196,6 +200,61 @@ class RecurrentOps:
         return self._scan(_SCAN_DELTA, src, q_col, k_col, v_col, H, G, D, Dv, log_decay, q_scale, beta_src,
                           beta_col, 0, 1.0, state, batch, write)
 
+    def head_delta_scan(self, src, q_col, k_col, v_col, H, G, D, Dv, gates, beta_col, decay_col, rates, decay_bias,
+                        state, batch, write):
+        """The delta rule of ``decay_scan`` with one decay a head and token,
+        exp(-exp(rates[h]) softplus(a + decay_bias[h])) with a at column ``decay_col`` + h of ``gates`` (float32
+        rows, which hold beta before its sigmoid at ``beta_col`` + h)."""
+        for name, v in (("rates", rates), ("decay biases", decay_bias)):
+            self._check(v, torch.float32, (H,), name)
+        return self._scan(_SCAN_DELTA_HEAD, src, q_col, k_col, v_col, H, G, D, Dv, None, 1.0, gates, beta_col, decay_col,
+                          1.0, state, batch, write, rates=rates, step_bias=decay_bias)
+
+    def selective_scan(self, u, proj, rank, N, step, step_t, step_bias, rates, skip, gate, gate_col, state, batch,
+                       write):
+        """The selective scan over ``u`` [T, C] (float32), a state of N places per channel.  ``proj`` (float32
+        rows) holds [step: rank | B: N | C: N]; dt = softplus(step ``step``^T + ``step_bias``), ``step`` [C, rank]
+        (``step_t`` its transpose); S'[n, c] = exp(``rates``[n, c] dt_c) S[n, c] + dt_c u_c B_n, y_c =
+        sum_n S'[n, c] C_n + ``skip``[c] u_c, times silu of column ``gate_col`` + c of ``gate`` (float32 rows).
+        The slot holds S as [N, C] from 0 on; a sequence whose first token is in the step starts from zero.
+        Returns rows [T, C] in the activation dtype.
+
+        Steps of one token a sequence are one launch (the step sizes' product included).  Longer ones: the step
+        sizes, then the scan in segments of SELECTIVE_SEGMENT tokens: what a segment leaves when it starts from
+        zero, what every segment starts from, and the read-outs."""
+        T, C = u.shape
+        self._f32_rows(u, "inputs")
+        width = self._f32_rows(proj, "projected rows")[1]
+        gate_stride = self._f32_rows(gate, "gate rows")[1]
+        if proj.shape[0] != T or gate.shape[0] != T or width < rank + 2 * N or not 0 <= gate_col <= gate_stride - C:
+            raise KernelError("selective_scan: the projected rows or the gates do not fit")
+        self._check(step, torch.float32, (C, rank), "step matrix")
+        self._check(step_t, torch.float32, (rank, C), "transposed step matrix")
+        self._check(step_bias, torch.float32, (C,), "step bias")
+        self._check(rates, torch.float32, (N, C), "rates")
+        self._check(skip, torch.float32, (C,), "skip")
+        self._sequences(batch, T)
+        slot_size = self._state(state, N * C)
+        S = batch.num_seqs
+        out = self._new((T, C))
+        lib = self._lazy("selective")
+        if batch.max_q_len == 1:
+            self._call(lib, "sl_selective_step", _p(u), C, _p(proj), width, rank, N, _p(step_t), _p(step_bias), _p(rates),
+                       _p(skip), _p(gate), gate_stride, gate_col, _p(state), _ll(slot_size), _p(batch.positions),
+                       _p(batch.tok_seq), _p(batch.state_slots), T, int(bool(write)), _p(out))
+            return out
+        dt = self.lowrank_expand(proj, 0, step, step_bias, "softplus")
+        seg = self.SELECTIVE_SEGMENT
+        segs = -(-batch.max_q_len // seg)
+        part = sums = None
+        if segs > 1 and N <= 64:
+            part = self._new((S, segs, N, C), torch.float32)
+            sums = self._new((S, segs, C), torch.float32)
+        self._call(lib, "sl_selective_scan", _p(u), _p(dt), C, _p(proj), width, rank, N, _p(rates), _p(skip), _p(gate),
+                   gate_stride, gate_col, _p(state), _ll(slot_size), _p(batch.cu_q), _p(batch.positions),
+                   _p(batch.state_slots), S, T, batch.max_q_len, seg, int(bool(write)), _p(part), _p(sums), _p(out))
+        return out
+
     def mlstm_scan(self, buf, q_col, k_col, v_col, i_col, f_col, H, D, Dv, cap, q_scale, state, batch, write):
         """The matrix LSTM: i = cap tanh(i~ / cap), f = logsigmoid(cap tanh(f~ / cap)), m' = max(f + m, i),
         S' = e^(f + m - m') S + e^(i - m') k v^T, n' likewise with k; returns S'^T q / (max(|n' . q|,
@@ -255,7 +314,7 @@ class RecurrentOps:
         (``slots`` None: no write); q comes back as [T, H D] in the activation dtype.
         ``per_head``: q and k are normed head by head instead (gains of the same sizes, so a gain may
         differ from head to head).  ``values_are_keys``: there is no v in ``buf``; the values cached are the keys as they lie
-        in ``buf``, before norm and rotation (Dv = D).  ``conv`` = (taps [C, n], state, state_off, batch,
+        in ``buf``, before norm and rotation (Dv = D).  ``G`` 0: ``buf`` holds queries only.  ``conv`` = (taps [C, n], state, state_off, batch,
         write): q, k and v (the row's first C channels) first pass the short causal convolution of
         ``short_conv`` without bias and activation, in the same launch; the state's last inputs are
         renewed when ``write``."""
@@ -266,11 +325,14 @@ class RecurrentOps:
             stride, conv = buf.shape[1], None
         if values_are_keys and Dv != D:
             raise KernelError("projnorm_rope_store: keys that serve as values have the values' width")
-        if (q_gain is None) != (k_gain is None):
+        if (q_gain is None) != (k_gain is None) and G:
             raise KernelError("projnorm_rope_store: both gains or neither")
+        if not G and slots is not None:
+            raise KernelError("projnorm_rope_store: there are no keys to store")
         if q_gain is not None:
             self._check(q_gain, torch.float32, (H * D,), "q gain")
-            self._check(k_gain, torch.float32, (G * D,), "k gain")
+            if G:
+                self._check(k_gain, torch.float32, (G * D,), "k gain")
         cos = sin = None
         if rot:
             cos, sin = tables.cos, tables.sin
@@ -303,13 +365,14 @@ class RecurrentOps:
                 _p(batch.tok_seq), _p(batch.state_slots), batch.num_seqs, int(bool(write)))
 
     # ------------------------------------------------------- routed experts
-    def route_tokens(self, logits, experts, top, over_all=False, correction=None, scale=1.0, with_matrices=None):
+    def route_tokens(self, logits, experts, top, over_all=False, correction=None, scale=1.0, with_matrices=None,
+                     sigmoid=False):
         """The ``top`` largest of each row's first ``experts`` logits (float32; among equals the
         lower index) with the softmax over them, and the step's (token, choice) pairs sorted by
         expert for the grouped products.  ``over_all``: what is compared is the softmax over all
         ``experts`` logits plus ``correction`` [experts] (None: nothing), and a chosen expert's
         share is its softmax value over the sum of the chosen ones' (+ 1e-20), times ``scale``.
-        ``with_matrices``: only the first so many experts have matrices (the others get no row
+        ``sigmoid``: a chosen expert's share is the sigmoid of its logit.  ``with_matrices``: only the first so many experts have matrices (the others get no row
         tiles; ``routed_experts`` hands their input through)."""
         T, stride = self._f32_rows(logits, "router logits")
         n = T * top
@@ -329,7 +392,7 @@ class RecurrentOps:
         real = experts if with_matrices is None else int(with_matrices)
         self._call(self._lazy("routed"), "sl_route_tokens", _p(logits), stride, T, experts, top, _p(chosen),
                    _p(shares), _p(order), _p(place_of), _p(tiles), max_tiles, tile_rows, int(bool(over_all)),
-                   _p(correction), _c_float(scale), real)
+                   _p(correction), _c_float(scale), real, int(bool(sigmoid)))
         return Routing(chosen, shares, order, place_of, tiles, tile_rows)
 
     def prepare_expert_matrices(self, w, gated=False):
@@ -345,14 +408,15 @@ class RecurrentOps:
         return ExpertMatrices(tiled, w.shape, True)
 
     def routed_experts(self, x, routing, w_gate_up, w_down, base=None, activation="silu", gated=True,
-                       base_gate=None, base_gate_col=0, limit=0.0, pass_through=False):
+                       base_gate=None, base_gate_col=0, limit=0.0, pass_through=False, weigh_input=False):
         """sum over a token's choices of share * down_e(act(gate_e x) * up_e x), plus ``base``;
         ``w_gate_up`` [E, 2 ff, width] holds an expert's gate rows before its up rows, ``w_down``
         [E, width, ff].  ``gated`` False: an expert is down_e(act(up_e x)) and ``w_gate_up`` is
         [E, ff, width].  ``base_gate`` (float32 rows): ``base`` is multiplied by the sigmoid of
         base_gate[t, base_gate_col].  ``activation`` "clamped_swish" (gated only): with g = min(gate_e x,
         limit) and u = clamp(up_e x, -limit, limit) the product is g sigmoid(1.702 g) (u + 1).
-        ``pass_through``: a chosen expert beyond the E with matrices adds share * x.  Sums are
+        ``weigh_input``: a share multiplies its expert's input (the float32 sums of the first products)
+        instead of its output.  ``pass_through``: a chosen expert beyond the E with matrices adds share * x.  Sums are
         float32; what lies between the two products is rounded to the activation dtype."""
         code = activation_code(activation)
         if not isinstance(w_gate_up, ExpertMatrices):
@@ -388,15 +452,17 @@ class RecurrentOps:
         mid = self._new((n, ff))
         self._call(lib, "sl_grouped_product", _p(x), _p(routing.order), top, _p(w_gate_up.data),
                    _p(routing.tiles), int(w_gate_up.tiled), max_tiles, routing.tile_rows, ff, K, int(bool(gated)), code,
-                   _c_float(limit), _p(mid))
+                   _c_float(limit), _p(routing.shares) if weigh_input else None, _p(mid))
         y = self._new((n, K), torch.float32)
         self._call(lib, "sl_grouped_product", _p(mid), None, 1, _p(w_down.data), _p(routing.tiles),
-                   int(w_down.tiled), max_tiles, routing.tile_rows, K, ff, 0, 0, _c_float(0.0), _p(y))
+                   int(w_down.tiled), max_tiles, routing.tile_rows, K, ff, 0, 0, _c_float(0.0), None,
+                   _p(y))
         out = self._new((T, K))
         gate_at = None
         if base_gate is not None:
             gate_at = ctypes.c_void_p(base_gate.data_ptr() + 4 * base_gate_col)
-        self._call(lib, "sl_routed_combine", _p(y), _p(routing.place_of), _p(routing.shares), T, top, _p(base),
+        self._call(lib, "sl_routed_combine", _p(y), _p(routing.place_of),
+                   None if weigh_input else _p(routing.shares), T, top, _p(base),
                    gate_at, gate_stride, K, _p(out), _p(routing.chosen) if pass_through else None, E,
                    _p(x) if pass_through else None)
         return out

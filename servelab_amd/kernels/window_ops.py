@@ -61,13 +61,15 @@ class WindowOps:
         self._check(delta, self.act_dtype, tuple(resid.shape), "delta")
         self._call("norm", "sl_add_into", _p(resid), _p(delta), _ll(resid.numel()))
 
-    def add_layernorm(self, resid, deltas, weight, eps, rows=None):
+    def add_layernorm(self, resid, deltas, weight, eps, rows=None, bias=None):
         """resid += sum of ``deltas`` (in place, float32), then the layer norm of every row with
-        gain ``weight`` and no bias.  ``rows`` (int32): only those rows are normed and returned, and
+        gain ``weight`` and ``bias`` (None: no bias).  ``rows`` (int32): only those rows are normed and returned, and
         the stream is left as it is."""
         T, H = resid.shape
         self._check(resid, torch.float32, None, "residual stream")
         self._check(weight, torch.float32, (H,), "norm weight")
+        if bias is not None:
+            self._check(bias, torch.float32, (H,), "norm bias")
         ds = self._plain_deltas(deltas)
         for d in ds:
             self._check(d, self.act_dtype, (T, H), "delta")
@@ -78,7 +80,8 @@ class WindowOps:
         R = T if rows is None else rows.shape[0]
         out = self._new((R, H))
         self._call("norm", "sl_add_layernorm", _p(resid), _p(ds[0]) if ds else None,
-                   _p(ds[1]) if len(ds) > 1 else None, _p(rows), _p(weight), _p(out), R, H, _c_float(eps))
+                   _p(ds[1]) if len(ds) > 1 else None, _p(rows), _p(weight), _p(bias), _p(out), R, H,
+                   _c_float(eps))
         return out
 
     # ------------------------------------------------- one matrix per head
@@ -184,7 +187,7 @@ class WindowOps:
     # ------------------------------------------------------------ attention
     def window_attention(self, q, q_col, nh, nkv, Dk, Dv, k_cache, v_cache, page_size, block_tables,
                          batch, scale, window, keep_first=0, slopes=None, sinks=None, gate=None,
-                         gate_col=0, softcap=None, channel_gate=None, channel_gate_col=0):
+                         gate_col=0, softcap=None, channel_gate=None, channel_gate_col=0, chunk=None):
         """Attention of every token of the batch over its sequence's pages.  ``q`` [T, width]
         holds head h of a token at column ``q_col + h * Dk``; ``v_cache`` None: values are the
         first Dv channels of the key rows.  ``window`` (None: all keys) and ``keep_first``: the
@@ -192,7 +195,8 @@ class WindowOps:
         [nh]: slope_h * (i - j) is taken off the scaled score; ``sinks`` [nh]: exp(sink_h) joins
         the denominator; ``gate`` [T, width] with head h's gate at column ``gate_col + h``: the
         output is multiplied by its sigmoid.  ``softcap`` c: the scaled score s becomes
-        c tanh(s / c).  ``channel_gate`` (float32 rows [T, width]): the output's channel d of head h is
+        c tanh(s / c).  ``chunk`` C: key j is seen only if j // C = i // C (or j < keep_first).
+        ``channel_gate`` (float32 rows [T, width]): the output's channel d of head h is
         multiplied by the sigmoid of column ``channel_gate_col + h * Dv + d``.  Returns [T, nh * Dv]."""
         T = q.shape[0]
         S, max_pages = block_tables.shape
@@ -227,7 +231,9 @@ class WindowOps:
             channel_stride = channel_gate.shape[1] if channel_gate.dim() == 2 else 0
             if channel_gate.shape[0] != T or channel_gate_col < 0 or channel_gate_col + nh * Dv > channel_stride:
                 raise KernelError("window_attention: the channel gates do not fit their rows")
-        window = int(window or 0)
+        window, chunk = int(window or 0), int(chunk or 0)
+        if window < 0 or chunk < 0:
+            raise KernelError("window_attention: window and chunk must not be negative")
         # shares of the keys: for steps of single tokens only, by the number of keys a token can see
         # there; fixed by sizes that a captured step keeps.  (A prompt's tiles are not cut: measured at
         # 2,048 tokens, two shares a tile save 35 us of attention over four layers and their merging
@@ -235,7 +241,9 @@ class WindowOps:
         mfma = self._window_mfma_fits(q, q_col, Dk, Dv)
         nsplit = 1
         if batch.max_q_len == 1:
-            span = batch.max_ctx_len if not window else min(batch.max_ctx_len, window + int(keep_first))
+            span = batch.max_ctx_len
+            if window or chunk:
+                span = min(span, min(n for n in (window, chunk) if n) + int(keep_first))
             if mfma:
                 # a workgroup for every CU, a block of 32 keys a share at least
                 nsplit = max(1, min(self.WINDOW_MFMA_MAX_SHARES, span // 32, self._num_cus // max(1, S * nkv)))
@@ -259,7 +267,7 @@ class WindowOps:
         self._call(lib, name, _c_void_p(q.data_ptr() + q_col * item), q.shape[1], _p(k_cache),
                    _p(v_cache), _p(block_tables), max_pages, _p(batch.cu_q), _p(batch.positions),
                    S, batch.max_q_len, T, nh, nkv, Dk, Dv, page_size, _c_float(scale),
-                   _c_float(float(softcap or 0.0)), window,
+                   _c_float(float(softcap or 0.0)), window, chunk,
                    int(keep_first), _p(slopes), _p(sinks),
                    _c_void_p(gate.data_ptr() + gate_col * item) if gate is not None else None, gate_stride,
                    _c_void_p(channel_gate.data_ptr() + 4 * channel_gate_col) if channel_gate is not None else None,
