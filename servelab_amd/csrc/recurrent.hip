@@ -99,8 +99,8 @@ __global__ __launch_bounds__(256) void lowrank_tile_kernel(const float* __restri
       ws[r][row] = in && c0 + row < C ? w2[(size_t)(c0 + row) * rank + r0 + r] : 0.f;
     }
     __syncthreads();
-    const int n = min(LOW_STEP, rank - r0);
-    for (int r = 0; r < n; ++r) {
+#pragma unroll
+    for (int r = 0; r < LOW_STEP; ++r) {               // (zeros beyond the rank)
       const float4 x = *(const float4*)&xs[r][4 * tr], w = *(const float4*)&ws[r][4 * tc];
       const float xv[4] = {x.x, x.y, x.z, x.w}, wv[4] = {w.x, w.y, w.z, w.w};
 #pragma unroll
@@ -181,7 +181,30 @@ struct ShortConv {
 
 // The sum over the taps of channel c for the token at place i of its step, whose inputs lie at first ..; with
 // a.shift (i is 0) the slot moves on by one, read and rewritten by the one thread that has the channel.
+// (N taps: all inputs are asked for before the first is used)
+template <int N>
+__device__ __forceinline__ float conv_channel_taps(const ShortConv& a, int first, int i, bool fresh, float* past, int c) {
+  float x[N], w[N];
+#pragma unroll
+  for (int j = 0; j < N; ++j) {
+    const int idx = i - (N - 1) + j;
+    w[j] = a.w[(size_t)c * N + j];
+    if (idx >= 0) x[j] = a.buf[(size_t)(first + idx) * a.stride + a.col + c];
+    else x[j] = fresh ? 0.f : past[(size_t)(N - 1 + idx) * a.C + c];
+  }
+  float acc = a.bias != nullptr ? a.bias[c] : 0.f;
+#pragma unroll
+  for (int j = 0; j < N; ++j) acc += w[j] * x[j];
+  if (a.shift) {
+#pragma unroll
+    for (int j = 1; j < N; ++j) past[(size_t)(j - 1) * a.C + c] = x[j];
+  }
+  return acc;
+}
 __device__ __forceinline__ float conv_channel(const ShortConv& a, int first, int i, bool fresh, float* past, int c) {
+  if (a.taps == 4) return conv_channel_taps<4>(a, first, i, fresh, past, c);
+  if (a.taps == 3) return conv_channel_taps<3>(a, first, i, fresh, past, c);
+  if (a.taps == 2) return conv_channel_taps<2>(a, first, i, fresh, past, c);
   const int back = a.taps - 1;
   float acc = a.bias != nullptr ? a.bias[c] : 0.f;
   for (int j = 0; j < a.taps; ++j) {

@@ -21,36 +21,57 @@ constexpr float SEL_LOG2E = 1.4426950408889634f;
 // exp(rate dt) with the rate already in units of log 2
 __device__ __forceinline__ float sel_decay(float rate2, float dt) { return __builtin_amdgcn_exp2f(rate2 * dt); }
 
-constexpr int SEL_STEP_THREADS = 64;
+constexpr int SEL_PARTS = 4, SEL_STEP_KEEP = 8;
 
-// One wavefront per (token, 64 channels).
-__global__ __launch_bounds__(SEL_STEP_THREADS) void selective_step_kernel(
+// Four wavefronts per (token, 64 channels): each takes a quarter of the rank for the step size, then a quarter
+// of the places; the partial sums meet in LDS and are added in the wavefronts' order.
+__global__ __launch_bounds__(64 * SEL_PARTS) void selective_step_kernel(
     const float* __restrict__ u, int C, const float* __restrict__ proj, int width, int R, int N,
     const float* __restrict__ wt, const float* __restrict__ bias, const float* __restrict__ rates,
     const float* __restrict__ skip, const float* __restrict__ gate, int gate_stride, int gate_col,
     float* __restrict__ state, long long state_stride, const int* __restrict__ positions,
     const int* __restrict__ tok_seq, const int* __restrict__ slots, int write, act_t* __restrict__ out) {
+  __shared__ float zs[SEL_PARTS][64], ys[SEL_PARTS][64];
   const size_t t = blockIdx.x;
-  const int c = blockIdx.y * SEL_STEP_THREADS + threadIdx.x;
-  if (c >= C) return;
+  const int lane = threadIdx.x & 63, part = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+  const int at = blockIdx.y * 64 + lane;
+  const bool live = at < C;
+  const int c = live ? at : C - 1;                      // (a lane past the last channel computes it and stores nothing)
   const float* row = proj + t * width;                  // (the same for the whole wavefront)
-  float z = 0.f;
-#pragma unroll 8
-  for (int r = 0; r < R; ++r) z += row[r] * wt[(size_t)r * C + c];
-  const float dt = sel_softplus(z + bias[c]);
-  const float x = u[t * C + c], dx = dt * x;
+  const float *B = row + R, *Cn = row + R + N;
   const bool fresh = positions[t] == 0;
   float* S = state + (size_t)slots[tok_seq[t]] * state_stride + c;
-  const float *B = row + R, *Cn = row + R + N;
-  float y = 0.f;
-#pragma unroll 8
-  for (int n = 0; n < N; ++n) {
-    const float old = fresh ? 0.f : S[(size_t)n * C];
-    const float s = sel_decay(rates[(size_t)n * C + c] * SEL_LOG2E, dt) * old + dx * B[n];
-    if (write) S[(size_t)n * C] = s;
-    y += s * Cn[n];
+  float old[SEL_STEP_KEEP], rate[SEL_STEP_KEEP];        // the first places' values are on their way meanwhile
+#pragma unroll
+  for (int k = 0; k < SEL_STEP_KEEP; ++k) {
+    const int n = part + SEL_PARTS * k;
+    old[k] = n < N && !fresh ? S[(size_t)n * C] : 0.f;
+    rate[k] = n < N ? rates[(size_t)n * C + c] : 0.f;
   }
-  y += skip[c] * x;
+  const float x = u[t * C + c];
+  float z = 0.f;
+#pragma unroll 16
+  for (int r = part; r < R; r += SEL_PARTS) z += row[r] * wt[(size_t)r * C + c];
+  zs[part][lane] = z;
+  __syncthreads();
+  z = (zs[0][lane] + zs[1][lane]) + (zs[2][lane] + zs[3][lane]);
+  const float dt = sel_softplus(z + bias[c]);
+  const float dx = dt * x;
+  float y = 0.f;
+  auto place = [&](int n, float before, float r) {
+    const float s = sel_decay(r * SEL_LOG2E, dt) * before + dx * B[n];
+    if (write && live) S[(size_t)n * C] = s;
+    y += s * Cn[n];
+  };
+#pragma unroll
+  for (int k = 0; k < SEL_STEP_KEEP; ++k)
+    if (part + SEL_PARTS * k < N) place(part + SEL_PARTS * k, old[k], rate[k]);
+  for (int n = part + SEL_PARTS * SEL_STEP_KEEP; n < N; n += SEL_PARTS)
+    place(n, fresh ? 0.f : S[(size_t)n * C], rates[(size_t)n * C + c]);
+  ys[part][lane] = y;
+  __syncthreads();
+  if (part != 0 || !live) return;
+  y = ((ys[0][lane] + ys[1][lane]) + (ys[2][lane] + ys[3][lane])) + skip[c] * x;
   out[t * C + c] = from_f<act_t>(y * sel_silu(gate[t * gate_stride + gate_col + c]));
 }
 
@@ -63,16 +84,15 @@ extern "C" const char* sl_selective_step(const float* u, int C, const float* pro
   SL_CHECK(R + 2 * N <= width && gate_col >= 0 && gate_col + C <= gate_stride, "selective_step: the rows are too short");
   SL_CHECK((long long)N * C <= state_stride, "selective_step: the state does not fit its slot");
   if (T == 0) return nullptr;
-  selective_step_kernel<<<dim3(T, (C + SEL_STEP_THREADS - 1) / SEL_STEP_THREADS), SEL_STEP_THREADS, 0, stream>>>(
+  selective_step_kernel<<<dim3(T, (C + 63) / 64), 64 * SEL_PARTS, 0, stream>>>(
       u, C, proj, width, R, N, wt, bias, rates, skip, gate, gate_stride, gate_col, state, state_stride, positions,
       tok_seq, slots, write, (act_t*)out);
   return sl_launch_status();
 }
 
-// A thread takes a channel of a (sequence, segment); NB places of its state (all of them, or the NB from n0
-// on: `more`).  READ: read-outs are formed; they are finished (skip, gate, rounding) by the last group of
-// places, which the groups before hand their sums in `acc`.
-//   PASS 0: from zero, into part and sums.   PASS 1: from part (segs > 1) or the slot, read-outs.
+// A thread takes a channel of a (sequence, segment) with its N places: NB exactly (EXACT) or at most.
+//   PASS 0: from zero, what it leaves into part and sums.
+//   PASS 1: from part (several segments) or the slot, read-outs, gate; one segment: the state into the slot.
 template <int NB, bool EXACT, int PASS>
 __global__ __launch_bounds__(64) void selective_segment_kernel(
     const float* __restrict__ u, const float* __restrict__ dts, int C, const float* __restrict__ proj, int width,
