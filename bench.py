@@ -220,9 +220,38 @@ def kelutar_configs(shape, layers, window, positions):
     return kelutar, vekanex_configs(shape, layers)[0]
 
 
+def lotinex_configs(shape, layers, window):
+    """(Lotinex config.json, Vekanex config.json) of equal size: Vekanex is the design nearest to it (a delta
+    rule with a matrix per head, an attention normed over its projection beside a second mixer, gated routed
+    experts).  Lotinex's layers come in the order delta rule (dense feed-forward), attention over a window
+    beside a selective scan (experts), attention in chunks (dense), attention over the keys of the layer
+    before it (experts), in a stream of four copies; the delta rule has the heads of Vekanex's, the scan twice the
+    width with 16 places a channel, 64 experts of which a token takes 8, without a shared one; windows and
+    chunks of --design-window tokens."""
+    z, v = DESIGN_SHAPES[shape], VEKANEX_SHAPES[shape]
+    w, H, D = z["width"], v["memory_heads"], v["memory_dim"]
+    dense = {"kind": "dense", "ff": z["ff"]}
+    moe = {"kind": "moe", "router": {"experts": v["experts"], "top": v["top"]}, "expert": {"ff": v["expert_ff"]}}
+    heads = {"heads": z["heads"], "kv_heads": z["kv_heads"], "dim": z["dim"], "vdim": z["dim"],
+             "scale": z["dim"] ** -0.5, "mask": {"size": window}}
+    delta = {"heads": 2 * H, "kv_heads": H, "dim": D, "vdim": v["memory_vdim"] // 2, "conv": 4}
+    chunked = dict(heads, rot={"base": 5e5, "dims": z["dim"]})
+    sides = {"left": dict(heads, softcap=50.0, conv=4, rot={
+                "base": 5e5, "dims": z["dim"] // 2, "scaling": {"factor": 8.0, "original": 8192, "fast": 32.0, "slow": 1.0}}),
+             "right": {"inner": 2 * w, "state": 16, "dt_rank": w // 16, "conv": 4}}
+    listed = []
+    for i in range(layers):
+        listed.append([{"type": "delta", "mixer": delta, "mlp": dense}, {"type": "parallel", "mixer": sides, "mlp": moe},
+                       {"type": "attention", "mixer": chunked, "mlp": dense},
+                       {"type": "attention", "mixer": dict(chunked, kv_from=i - 1), "mlp": moe}][i % 4])
+    lotinex = {"architecture": "Lotinex", "width": w, "vocab": z["vocab"], "streams": 4, "norm": {"eps": 1e-5},
+               "embedding": {"scale": w ** 0.5}, "torch_dtype": "bfloat16", "layers": listed}
+    return lotinex, vekanex_configs(shape, layers)[0]
+
+
 def compare_designs(args):
     """Prefill and decode throughput of the design named by --design beside the Qwen2 decoder of equal
-    size (Futezen and Kelutar: beside the Vekanex decoder of equal size; Vunadra: beside the Futezen one),
+    size (Futezen, Kelutar and Lotinex: beside the Vekanex decoder of equal size; Vunadra: beside the Futezen one),
     at each of --design-shapes: one JSON line, tokens per second each."""
     import torch
     import servelab_amd  # noqa: F401
@@ -236,9 +265,10 @@ def compare_designs(args):
                       "prefill_chunk": args.prefill_chunk, "page_size": page}, "shapes": {}}
     for shape in args.design_shapes.split(","):
         row = {}
-        other = {"futezen": "vekanex", "kelutar": "vekanex", "vunadra": "futezen"}.get(args.design, "qwen2")
+        other = {"futezen": "vekanex", "kelutar": "vekanex", "lotinex": "vekanex", "vunadra": "futezen"}.get(args.design, "qwen2")
         pair = kelutar_configs(shape, args.design_layers, args.design_window,
                                2 * max(args.context, args.prefill_tokens)) if args.design == "kelutar" else \
+            lotinex_configs(shape, args.design_layers, args.design_window) if args.design == "lotinex" else \
             vunadra_configs(shape, args.design_layers, args.design_window) if args.design == "vunadra" else \
             futezen_configs(shape, args.design_layers) if args.design == "futezen" else \
             vekanex_configs(shape, args.design_layers) if args.design == "vekanex" else \
@@ -408,7 +438,7 @@ def main():
     ap.add_argument("--no-prefill", action="store_true")
     ap.add_argument("--no-tune", action="store_true",
                     help="leave the library's default kernel choice for the prompt products")
-    ap.add_argument("--design", default="", choices=["", "topelorn", "vekanex", "futezen", "vunadra", "kelutar"],
+    ap.add_argument("--design", default="", choices=["", "topelorn", "vekanex", "futezen", "vunadra", "kelutar", "lotinex"],
                     help="instead of the default workload: prefill and decode throughput of this design "
                          "beside the Qwen2 decoder of equal size")
     ap.add_argument("--design-shapes", default="3b,7b", help="comma-separated: " + ", ".join(sorted(DESIGN_SHAPES)))
